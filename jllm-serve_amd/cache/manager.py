@@ -9,7 +9,8 @@ What is different: the reference has one group and refuses models whose layers d
 (model/Decoder.java:40-49). Here every cache-owning run of the layer schedule declares a ``PageSpec``
 (named per-position tensors and a window; ``KvSpec`` makes the one of attention); runs with equal specs form a group with its own pool, storage and block table per request. A group with
 a window gives pages back as soon as every position in them is older than any later query can see
-(model/Attention.java:68-71: the query at p sees keys from max(0, p + 1 - window)). Beside the pages
+(model/Attention.java:68-71: the query at p sees keys from max(0, p + 1 - window)); so does a group whose positions are
+read within chunks of the sequence only, when a chunk is complete. Beside the pages
 there are fixed-size state slots: one index per live request into per-run state tensors.
 
 With ``prefix_share`` the full pages of a request are published in a prefix tree (cache/prefix.py) and a
@@ -58,11 +59,25 @@ class PageSpec:
     rows: Tuple[CacheRow, ...]
     window: int = 0  # 0 = all earlier positions stay visible
     keep_first: int = 0  # with a window: the positions before this one stay visible too, and their pages are never given back
+    chunk: int = 0  # in place of a window: a position is read by the positions of its own chunk of this many (from 0) only
 
     def __post_init__(self):
         names = [r.name for r in self.rows]
         if not names or len(set(names)) != len(names):
             raise ValueError(f"a page spec needs rows with distinct names, got {names}")
+        if self.chunk < 0 or (self.chunk and self.window):
+            raise ValueError(f"a page spec has a window or chunks, got {self.window} and {self.chunk}")
+
+    @property
+    def forgets(self) -> bool:
+        """Whether there are positions that no later position reads."""
+        return self.window > 0 or self.chunk > 0
+
+    def first_needed(self, length: int) -> int:
+        """The oldest position (kept first ones aside) that any position >= ``length`` still reads."""
+        if self.chunk > 0:
+            return length // self.chunk * self.chunk
+        return max(0, length + 1 - self.window) if self.window > 0 else 0
 
 
 def KvSpec(kv_heads: int, head_dim: int, window: int = 0) -> PageSpec:
@@ -181,8 +196,9 @@ class CacheManager:
         self.requests: Dict[object, RequestCache] = {}
         self.pages_given_back_by_window = 0
         self.sharing_refused = ""
-        if prefix_share and any(g.spec.window > 0 for g in self.groups):
-            self.sharing_refused = "a group of layers has a window"
+        if prefix_share and any(g.spec.forgets for g in self.groups):
+            self.sharing_refused = "a group of layers has a window" if any(g.spec.window > 0 for g in self.groups) else \
+                "a group of layers reads within chunks"
         elif prefix_share and any(p.state is not None for p in plans):
             self.sharing_refused = "a layer keeps per-request state"
         elif prefix_share and not self.groups:
@@ -235,7 +251,7 @@ class CacheManager:
 
     def _first_needed(self, g: KvGroup, length: int) -> int:
         """The oldest position any query at position >= length still sees in group g."""
-        return max(0, length + 1 - g.spec.window) if g.spec.window > 0 else 0
+        return g.spec.first_needed(length)
 
     def pages_needed(self, rid, n: int) -> List[int]:
         """Pages each group would have to allocate for the next n tokens of the request."""
@@ -338,7 +354,7 @@ class CacheManager:
         rc.length += n
         assert all(len(t) * self.page_size >= rc.length for t in rc.tables), "commit beyond the pages begun"
         for gi, g in enumerate(self.groups):
-            if g.spec.window <= 0:
+            if not g.spec.forgets:
                 continue
             first = self._first_needed(g, rc.length)
             whole = first // self.page_size  # table entries wholly before `first`
@@ -362,7 +378,7 @@ class CacheManager:
         keep = -(-length // self.page_size)
         for gi, g in enumerate(self.groups):
             kept = -(-g.spec.keep_first // self.page_size)
-            if g.spec.window > 0 and max(self._first_needed(g, length) // self.page_size, kept) < rc.released[gi]:
+            if g.spec.forgets and max(self._first_needed(g, length) // self.page_size, kept) < rc.released[gi]:
                 raise ValueError("the window of this group has already given back pages the shorter sequence needs")
             while len(rc.tables[gi]) > keep:
                 p = rc.tables[gi].pop()
@@ -522,7 +538,7 @@ class CacheManager:
     def stats(self) -> dict:
         return {
             "page_size": self.page_size,
-            "groups": [{"runs": len(g.runs), "window": g.spec.window, "pages": g.pool.num_pages,
+            "groups": [{"runs": len(g.runs), "window": g.spec.window, "chunk": g.spec.chunk, "pages": g.pool.num_pages,
                         "used": g.pool.used_pages, "free": g.pool.free_pages, "high_water": g.pool.high_water,
                         "allocations": g.pool.allocations} for g in self.groups],
             "requests": len(self.requests),

@@ -71,9 +71,11 @@ class LearnedPositionSpec:
 
 @dataclass(frozen=True)
 class NormSpec:
-    """RMSNorm with a plain gain (no 1+w) and the model's eps (model/Families.java:663, :793)."""
+    """RMSNorm with a plain gain (no 1+w) and the model's eps (model/Families.java:663, :793). ``one_plus``: the stored
+    weight w means a gain of 1 + w (formed in fp32)."""
 
     eps: float
+    one_plus: bool = False
     kind: str = "rmsnorm"
 
 
@@ -220,6 +222,7 @@ class WideAttentionNames:
     lambda_q: Tuple[str, ...] = ("lq1", "lq2")  # differential attention: the vectors whose products give lambda
     lambda_k: Tuple[str, ...] = ("lk1", "lk2")
     sink: str = "sink"
+    temp: str = "temp"
 
 
 @dataclass(frozen=True)
@@ -239,7 +242,12 @@ class WideAttentionSpec:
     tensors ``<q>.norm`` / ``<k>.norm``). ``window`` > 0: the query at p sees keys p + 1 - window .. p, and, with
     ``keep_first``, also the keys at positions before ``keep_first`` (each still at the position it was written at). ``sink``: a
     learned number per head (tensor ``sink`` [heads]) whose exponential joins the softmax's denominator as it is: nothing
-    is looked up for it, nothing is added to the weighted sum, and the scale does not touch it."""
+    is looked up for it, nothing is added to the weighted sum, and the scale does not touch it. ``chunk`` > 0 (in place
+    of a window): the sequence is cut into chunks of that many positions counted from 0, and the query at p sees the keys
+    of its own chunk up to p. ``tied_values``: there is no value projection, the values are the keys as projected, before
+    any norm or rotation (``vdim`` is ``dim``). ``head_temp``: head h's scores are multiplied by the h-th number of the
+    tensor ``temp`` [heads]. ``distance_bias``: with s_h = 2^(-8 (h + 1) / heads), s_h times the distance between query
+    and key is taken off head h's scores."""
 
     heads: int
     kv_heads: int
@@ -260,6 +268,10 @@ class WideAttentionSpec:
     keep_first: int = 0
     sink: bool = False
     gate_per_head: bool = False
+    chunk: int = 0
+    tied_values: bool = False
+    head_temp: bool = False
+    distance_bias: bool = False
     names: WideAttentionNames = WideAttentionNames()
     kind: str = "wide_attention"
 
@@ -350,13 +362,53 @@ class StateSpaceSpec:
 
 
 @dataclass(frozen=True)
+class LinearAttentionNames:
+    """Tensor names of a linear-attention mixer under its prefix."""
+
+    q: str = "q"
+    k: str = "k"
+    v: str = "v"
+    gate: str = "g"
+    norm: str = "norm"
+    o: str = "o"
+
+
+@dataclass(frozen=True)
+class LinearAttentionSpec:
+    """Linear attention with a fixed decay per head: a recurrent mixer without a softmax or a denominator. q and k of
+    heads x ``dim`` and v of heads x ``vdim`` are projections of the input, each through ``activation`` (None or "silu");
+    ``position``: index of a rotary table applied to q and k (half pairing, the first rotary_dim entries of every head)
+    or None; k is multiplied by ``k_scale``. Per head S <- decay_h S + k v^T with S [dim, vdim] from zero, o = S^T q.
+    ``norm`` "head": every head's o is divided by its root mean square (no weight); "whole": the concatenated heads are
+    RMS-normed together with a weight (tensor ``norm`` [heads x vdim]); ``eps`` inside the root. Then times
+    ``gate_fn``(W_g h), "silu" or "sigmoid", and through W_o."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: Tuple[float, ...]
+    eps: float
+    activation: Optional[str] = None
+    position: Optional[int] = None
+    k_scale: float = 1.0
+    norm: str = "head"
+    gate_fn: str = "silu"
+    names: LinearAttentionNames = LinearAttentionNames()
+    kind: str = "linear_attention"
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Mixers side by side on the same input: the result is the sum of ``scales[i]`` times branch i's output. Branch
-    i's tensors lie under the mixer's prefix + ``prefixes[i]``. At most one branch may own pages."""
+    i's tensors lie under the mixer's prefix + ``prefixes[i]``. At most one branch may own pages. ``out_norms`` (one
+    tensor name per branch, under the mixer's prefix): branch i's output is first RMS-normed over the model width with
+    that plain weight and ``out_eps``."""
 
     branches: Tuple[Any, ...]
     scales: Tuple[float, ...]
     prefixes: Tuple[str, ...]
+    out_norms: Tuple[str, ...] = ()
+    out_eps: float = 0.0
     kind: str = "parallel"
 
 
@@ -473,6 +525,9 @@ class LayerSpec:
 
     ``arrangement`` "prenorm": x += mixer(norm(x)); x += ffn(norm(x)) (model/LayerSpec.java:18-19,
     cpu/CpuBackend.java:959-969). "parallel": with h = norm(x), x += mixer(h) + ffn(h): one norm, both sublayers read it.
+    "postnorm": x += norm(mixer(x)); x += norm(ffn(x)): the sublayers read the stream itself, their outputs are normed.
+    ``token_shift`` (a tensor name under the prefix, [hidden]; the postnorm arrangement takes it): what the mixer reads, h_t,
+    is first replaced by h_t + shift (h_(t-1) - h_t), element by element, with zeros before a sequence's first token.
     ``ffn`` None: the layer has no feed-forward (and no second norm). ``prefix`` is the tensor-name prefix of the layer's weights; the names under it
     are data of the specs (here the two norms', in the mixer's and feed-forward's specs theirs), so a checkpoint
     that names or stacks its tensors differently is a matter of the parser.
@@ -490,6 +545,7 @@ class LayerSpec:
     norm_mixer_out_name: str = ""
     norm_ffn_out_name: str = ""
     mixer_prefix: str = ""  # under the layer's prefix, for mixers whose tensor names are relative to it
+    token_shift: str = ""
     # arrangement "hyper": the stream has ``streams`` copies per row; sublayer q reads u = sum_s in[s] x_s, and all
     # streams are rewritten at once, x_t <- sum_s mix[s, t] x_s + out[t] * sublayer(norm(u)), with the tensors
     # ``<prefix>.<hyper_names[q]>.in`` [streams], ``.out`` [streams], ``.mix`` [streams, streams] (row: the stream read, column: the stream written)

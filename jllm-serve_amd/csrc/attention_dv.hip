@@ -8,7 +8,8 @@
 //                    whole of q and the whole of k (or over every head alone, with gains shared by the heads); optional
 //                    rotation of the pairs (2i, 2i + 1) (or (i, i + rot_dims / 2)) among the first rot_dims entries of
 //                    every q and k head by the row's position; optional q *= 1 + coef * ln(floor((p + 1) / every) + 1);
-//                    q back in place, k and v into the row's place in the cache
+//                    and q times a number per head; q back in place, k and v into the row's place in the cache (with
+//                    tied values there are no v columns: the values are the k columns as they came)
 //   attention_dv     one workgroup of four waves per (row, query slot). A query slot is one score map of one head: with
 //                    M maps per head and H heads over G key/value heads there are H * M query slots and G * M key slots;
 //                    query slot s reads key slot (s / (M * H / G)) * M + s % M and value head s / (M * H / G). Scores
@@ -16,8 +17,10 @@
 //                    to absolute positions, wave w takes the blocks with c % 4 == w, the four waves' results are merged
 //                    in wave order: a row's result depends only on its own position and keys. With a window the query
 //                    at p sees keys p + 1 - window .. p and, with keep_first, the keys before keep_first (the blocks
-//                    between them are passed over: their pages may be gone). A sink per head adds exp(sink) to the
-//                    denominator and nothing to the sum
+//                    between them are passed over: their pages may be gone). With chunks the query at p sees the keys
+//                    of its own chunk of the sequence (positions p / chunk * chunk .. p). A slope per head takes slope *
+//                    (p - j) off the score of the key at j. A sink per head adds exp(sink) to the denominator and
+//                    nothing to the sum
 //   heads_finish     per (row, head): with two maps o = a1 - lambda * a2; optionally o / sqrt(mean(o^2) + eps) * gain;
 //                    optionally times sigmoid(gate) or silu(gate) (a gate per channel or one per head), times a
 //                    constant; written as the output product's
@@ -38,7 +41,8 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
     T* __restrict__ qkv, int ld, const int* __restrict__ positions, const int* __restrict__ slots, int q_slots, int k_slots,
     int v_heads, int dk, int dv, const TG* __restrict__ gq, const TG* __restrict__ gk, float eps,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot_dims, float temp_coef, int temp_every,
-    T* __restrict__ kcache, T* __restrict__ vcache, int page_size, int norm_per_head, int pair_halves) {
+    T* __restrict__ kcache, T* __restrict__ vcache, int page_size, int norm_per_head, int pair_halves,
+    const float* __restrict__ head_mul, int maps, int v_off) {
   extern __shared__ float sm[];  // q and k of the row
   __shared__ float red[PREP_THREADS / 64];
   const int t = blockIdx.x;
@@ -84,7 +88,8 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
   }
   float temp = 1.0f;
   if (temp_every > 0) temp = 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f);
-  for (int i = threadIdx.x; i < nq; i += PREP_THREADS) stf(row, i, sm[i] * temp);
+  for (int i = threadIdx.x; i < nq; i += PREP_THREADS)
+    stf(row, i, sm[i] * (head_mul ? temp * head_mul[i / (dk * maps)] : temp));
   const int slot = slots ? slots[t] : -1;
   if (slot < 0) return;  // a row that stores nothing (padding of a step of fixed size; a run that reads another's cache)
   const int page = slot / page_size, off = slot % page_size;
@@ -94,7 +99,7 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
   }
   for (int i = threadIdx.x; i < nv; i += PREP_THREADS) {
     const int h = i / dv, e = i % dv;
-    vcache[(((size_t)page * v_heads + h) * page_size + off) * dv + e] = row[nq + nk + i];
+    vcache[(((size_t)page * v_heads + h) * page_size + off) * dv + e] = row[v_off + i];
   }
 }
 
@@ -102,10 +107,13 @@ extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, cons
                                 int q_slots, int k_slots, int v_heads, int dk, int dv, const void* gq, const void* gk,
                                 int gain_dtype, float eps, const float* cos_t, const float* sin_t, int rot_dims,
                                 float temp_coef, int temp_every, void* kcache, void* vcache, int page_size,
-                                int norm_per_head, int pair_halves, hipStream_t stream) {
+                                int norm_per_head, int pair_halves, const float* head_mul, int maps, int tied_values,
+                                hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (q_slots <= 0 || k_slots <= 0 || v_heads <= 0 || dk <= 0 || dv <= 0) JLLM_FAIL("qkv_prepare: sizes %d %d %d %d %d", q_slots, k_slots, v_heads, dk, dv);
-  if (ld < (q_slots + k_slots) * dk + v_heads * dv) JLLM_FAIL("qkv_prepare: rows of %d entries are shorter than q, k and v", ld);
+  if (tied_values && (v_heads != k_slots || dv != dk)) JLLM_FAIL("qkv_prepare: values that are the keys take %d heads of %d, got %d of %d", k_slots, dk, v_heads, dv);
+  if (ld < (q_slots + k_slots) * dk + (tied_values ? 0 : v_heads * dv)) JLLM_FAIL("qkv_prepare: rows of %d entries are shorter than q, k and v", ld);
+  if (maps <= 0 || q_slots % maps) JLLM_FAIL("qkv_prepare: %d query slots with %d maps per head", q_slots, maps);
   if ((gq == nullptr) != (gk == nullptr)) JLLM_FAIL("qkv_prepare: the norm takes gains for both q and k");
   if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims && (!cos_t || !sin_t))) JLLM_FAIL("qkv_prepare: a rotary width of %d for heads of %d", rot_dims, dk);
   if (page_size <= 0) JLLM_FAIL("qkv_prepare: page_size %d", page_size);
@@ -115,7 +123,8 @@ extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, cons
     JLLM_DISPATCH_1(gain_dtype, TG, {
       qkv_prepare_kernel<T, TG><<<n_tokens, PREP_THREADS, smem, stream>>>(
           (T*)qkv, ld, positions, slots, q_slots, k_slots, v_heads, dk, dv, (const TG*)gq, (const TG*)gk, eps, cos_t, sin_t,
-          rot_dims, temp_coef, temp_every, (T*)kcache, (T*)vcache, page_size, norm_per_head, pair_halves);
+          rot_dims, temp_coef, temp_every, (T*)kcache, (T*)vcache, page_size, norm_per_head, pair_halves, head_mul, maps,
+          tied_values ? q_slots * dk : (q_slots + k_slots) * dk);
     })
   })
   JLLM_CHECK_LAUNCH("qkv_prepare");
@@ -129,7 +138,8 @@ __global__ __launch_bounds__(64 * ADV_WAVES) void attention_dv_generic_kernel(
     const T* __restrict__ q, int ldq, TO* __restrict__ out, int ldo, const T* __restrict__ kcache,
     const T* __restrict__ vcache, const int* __restrict__ block_table, int max_blocks, const int* __restrict__ row_req,
     const int* __restrict__ positions, int q_slots, int maps, int per_kv, int dk, int dv, int page_size, int window,
-    float scale, float softcap, int keep_first, const float* __restrict__ sinks) {
+    float scale, float softcap, int keep_first, const float* __restrict__ sinks, int chunk,
+    const float* __restrict__ slopes) {
   extern __shared__ float smem[];
   float* qs = smem;       // dk
   float* mg = smem + dk;  // ADV_WAVES x (2 + dv)
@@ -140,7 +150,8 @@ __global__ __launch_bounds__(64 * ADV_WAVES) void attention_dv_generic_kernel(
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int pos = positions[t];
   const int* tbl = block_table + (size_t)row_req[t] * max_blocks;
-  const int first = window > 0 ? max(0, pos + 1 - window) : 0;
+  const int first = window > 0 ? max(0, pos + 1 - window) : chunk > 0 ? pos / chunk * chunk : 0;
+  const float slope = slopes ? slopes[s / maps] : 0.f;
   for (int i = threadIdx.x; i < dk; i += 64 * ADV_WAVES) qs[i] = ldf(q + (size_t)t * ldq + (size_t)s * dk, i);
   __syncthreads();
   const int nacc = (dv + 63) >> 6;
@@ -167,6 +178,7 @@ __global__ __launch_bounds__(64 * ADV_WAVES) void attention_dv_generic_kernel(
       for (int i = 0; i < dk; ++i) d = fmaf(qs[i], ldf(kr, i), d);
       sc = d * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+      sc -= slope * (float)(pos - kj);
     }
     const float m_new = fmaxf(m, wave_max(sc));
     const float p = valid ? expf(sc - m_new) : 0.f;
@@ -229,8 +241,10 @@ extern "C" int jllm_attention_dv_generic(const void* q, int ldq, int dtype, void
                                          const void* kcache, const void* vcache, const int* block_table, int max_blocks,
                                          const int* row_req, const int* positions, int n_tokens, int heads, int kv_heads,
                                          int maps, int dk, int dv, int page_size, int window, float scale, float softcap,
-                                         int keep_first, const float* sinks, hipStream_t stream) {
+                                         int keep_first, const float* sinks, int chunk, const float* slopes,
+                                         hipStream_t stream) {
   if (n_tokens <= 0) return 0;
+  if (chunk < 0 || (chunk > 0 && window > 0)) JLLM_FAIL("attention: chunks of %d beside a window of %d", chunk, window);
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || maps <= 0) JLLM_FAIL("attention: %d query heads over %d kv heads with %d maps", heads, kv_heads, maps);
   if (dk <= 0 || dv <= 0 || dv > 64 * ADV_MAX_ACC || dk > 4096) JLLM_FAIL("attention: key size %d, value size %d (this kernel takes values up to %d)", dk, dv, 64 * ADV_MAX_ACC);
   const int q_slots = heads * maps;
@@ -243,7 +257,7 @@ extern "C" int jllm_attention_dv_generic(const void* q, int ldq, int dtype, void
     JLLM_DISPATCH_1(out_dtype, TO, {
       attention_dv_generic_kernel<T, TO><<<grid, 64 * ADV_WAVES, smem, stream>>>(
           (const T*)q, ldq, (TO*)out, ldo, (const T*)kcache, (const T*)vcache, block_table, max_blocks, row_req, positions,
-          q_slots, maps, maps * (heads / kv_heads), dk, dv, page_size, window, scale, softcap, keep_first, sinks);
+          q_slots, maps, maps * (heads / kv_heads), dk, dv, page_size, window, scale, softcap, keep_first, sinks, chunk, slopes);
     })
   })
   JLLM_CHECK_LAUNCH("attention_dv_generic");

@@ -9,7 +9,10 @@
 // are in flight while this one is multiplied); places outside the tile's visible range are stored as zeros and
 // their table entries are never read. With kept first keys (keys before `keep_first` stay visible whatever the window)
 // a tile's blocks are numbered: first the blocks of the kept keys that lie wholly before the window's first block, then
-// the window's; a sink per head adds exp(sink) to the denominator where it is finished (here, or in the merge).
+// the window's; a sink per head adds exp(sink) to the denominator where it is finished (here, or in the merge). With
+// chunks (in place of a window) the query at p sees positions p / chunk * chunk .. p: a tile's keys start with its first
+// row's chunk, and a wave passes over the blocks in front of its own rows' chunks. A slope per head takes slope *
+// (query position - key position) off the scores in front of the softmax.
 //
 // Each wave computes the transposed scores S^T[key][row] = K Q^T (v_mfma_f32_32x32x16_bf16, A = K from LDS, B = Q
 // in registers), so a lane owns one query row: maximum and sum are in-lane reductions plus one exchange between the
@@ -36,7 +39,7 @@ __global__ __launch_bounds__(256, (DK16 <= 8 && DB <= 4) ? 2 : 1) void attention
     const bf16_t* __restrict__ vc, const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tiles,
     const int* __restrict__ positions, int maps, int per_kv, int k_slots, int v_heads, int dv, int page_shift, int window,
     float scale, float softcap, float* __restrict__ partial, int per_split, int share, int q_slots, int keep_first,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, int chunk, const float* __restrict__ slopes) {
   constexpr int DK = DK16 * 16;
   constexpr int DVP = DB * 32;
   constexpr int KLD = DK + 8;
@@ -63,13 +66,16 @@ __global__ __launch_bounds__(256, (DK16 <= 8 && DB <= 4) ? 2 : 1) void attention
   const int wq = share ? 0 : wave * 32 + qi;                    // the lane's row within the tile
   const bool lane_on = share ? (wave == 0 && qi < share) : (wq < nrows);
   const int pos_q = pos0 + min(wq, nrows - 1);
-  const int first_q = window > 0 ? max(0, pos_q + 1 - window) : 0;
+  // the first key that the query at p sees beside the kept ones (it never moves back as p grows)
+  auto first_key = [&](int p) { return window > 0 ? max(0, p + 1 - window) : chunk > 0 ? p / chunk * chunk : 0; };
+  const int first_q = first_key(pos_q);
   const int* tbl = block_table + (size_t)req * max_blocks;
-  const int k_lo = window > 0 ? max(0, pos0 + 1 - window) : 0;
+  const int k_lo = first_key(pos0);
   const int k_hi = pos0 + nrows - 1;
   const int wave_lo_pos = pos0 + min(nrows - 1, wave * 32);
   const int wave_hi = pos0 + min(nrows - 1, wave * 32 + 31);
-  const int wave_first = window > 0 ? max(0, wave_hi + 1 - window) : 0;
+  const int wave_first = first_key(wave_hi);
+  const int wave_lo_first = first_key(wave_lo_pos);
   const bool wave_on = share ? wave == 0 : wave * 32 < nrows;
   u32x4 qf[DK16];
   {
@@ -158,7 +164,9 @@ __global__ __launch_bounds__(256, (DK16 <= 8 && DB <= 4) ? 2 : 1) void attention
     for (int e = 0; e < 16; ++e) o[db][e] = 0.f;
   float m = -INFINITY, l = 0.f;
   const float log2e = 1.4426950408889634f;
-  const float sl = softcap > 0.f ? log2e : scale * log2e;  // capped scores are final; raw ones are scaled in the exponent
+  const float raw_sl = softcap > 0.f ? log2e : scale * log2e;  // capped scores are final; raw ones are scaled in the exponent
+  const float slope2 = slopes ? slopes[s / maps] * log2e : 0.f;
+  const float sl = slopes ? 1.0f : raw_sl;  // with a slope the scores are brought to the exponent's unit where it is taken off
   const float cap_in = softcap > 0.f ? 2.0f * log2e * scale / softcap : 0.f;
   // beyond a tile's last block the block numbers name keys past k_hi, whose table entries are never read
   load_pages(block_keys(it_first));
@@ -174,7 +182,7 @@ __global__ __launch_bounds__(256, (DK16 <= 8 && DB <= 4) ? 2 : 1) void attention
       load_block(block_keys(it_first + it + 1));
       load_pages(block_keys(it_first + it + 2));
     }
-    if (wave_on && kt <= wave_hi) {
+    if (wave_on && kt <= wave_hi && (kt + AT_KEYS > wave_lo_first || kt < kept)) {
       const bf16_t* Kb = Ks + buf * KSZ;
       const bf16_t* Vb = Vs + buf * VSZ + v_lane;
       floatx16 sc[2];
@@ -192,6 +200,14 @@ __global__ __launch_bounds__(256, (DK16 <= 8 && DB <= 4) ? 2 : 1) void attention
 #pragma unroll
           for (int e = 0; e < 16; ++e)
             sc[kb][e] = softcap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sc[kb][e] * cap_in)));
+      }
+      if (slopes) {  // the distance from the query to the key times the head's slope
+        const int dist0 = kt + half * 4 - pos_q;
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+          for (int e = 0; e < 16; ++e)
+            sc[kb][e] = fmaf(sc[kb][e], raw_sl, slope2 * (float)(dist0 + kb * 32 + 8 * (e >> 2) + (e & 3)));
       }
       const bool all_visible = kt + AT_KEYS - 1 <= wave_lo_pos && (kt >= wave_first || kt + AT_KEYS <= kept);
       if (!all_visible) {
@@ -320,7 +336,8 @@ template <int DK16, int DB>
 static int launch_tiles(dim3 grid, hipStream_t stream, const bf16_t* q, int ldq, float* out, int ldo, const bf16_t* kc,
                         const bf16_t* vc, const int* block_table, int max_blocks, const int* tiles, const int* positions, int maps,
                         int per_kv, int k_slots, int v_heads, int dv, int page_shift, int window, float scale, float softcap,
-                        float* partial, int per_split, int share, int q_slots, int keep_first, const float* sinks) {
+                        float* partial, int per_split, int share, int q_slots, int keep_first, const float* sinks, int chunk,
+                        const float* slopes) {
   const size_t smem = (size_t)2 * AT_KEYS * ((DK16 * 16 + 8) + (DB * 32 + 32)) * sizeof(bf16_t);
   static bool raised = false;
   if (smem > 64 * 1024 && !raised) {
@@ -330,7 +347,7 @@ static int launch_tiles(dim3 grid, hipStream_t stream, const bf16_t* q, int ldq,
   }
   attention_dv_tiles_kernel<DK16, DB><<<grid, 256, smem, stream>>>(q, ldq, out, ldo, kc, vc, block_table, max_blocks, tiles, positions,
                                                                  maps, per_kv, k_slots, v_heads, dv, page_shift, window, scale, softcap,
-                                                                 partial, per_split, share, q_slots, keep_first, sinks);
+                                                                 partial, per_split, share, q_slots, keep_first, sinks, chunk, slopes);
   return 0;
 }
 
@@ -342,12 +359,14 @@ extern "C" int jllm_attention_dv_bf16(const void* q, int ldq, float* out, int ld
                                       const int* block_table, int max_blocks, const int* tiles, int n_tiles,
                                       const int* positions, int heads, int kv_heads, int maps, int dk, int dv, int page_size,
                                       int window, float scale, float softcap, int splits, int per_split, float* partial,
-                                      int n_rows, int defer_merge, int keep_first, const float* sinks, hipStream_t stream) {
+                                      int n_rows, int defer_merge, int keep_first, const float* sinks, int chunk,
+                                      const float* slopes, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || maps <= 0) JLLM_FAIL("attention: %d query heads over %d kv heads with %d maps", heads, kv_heads, maps);
   if ((dk & 15) || dk < 16 || dk > 256 || (dv & 7) || dv < 8 || dv > 256) return 1;
   if (!(scale > 0.f) || softcap < 0.f || keep_first < 0) return 1;  // the maximum is taken before the scale's sign could matter
   if ((ldq & 7) || (ldo & 3) || ((uintptr_t)q & 15) || ((uintptr_t)out & 15) || ((uintptr_t)kcache & 15) || ((uintptr_t)vcache & 15)) return 1;
+  if (chunk < 0 || (chunk > 0 && window > 0)) JLLM_FAIL("attention: chunks of %d beside a window of %d", chunk, window);
   if (page_size <= 0 || (page_size & (page_size - 1)) || n_tiles > 65535 || heads * maps > 65535) return 1;
   int page_shift = 0;
   while ((1 << page_shift) < page_size) ++page_shift;
@@ -361,7 +380,7 @@ extern "C" int jllm_attention_dv_bf16(const void* q, int ldq, float* out, int ld
   int rc = 1;
 #define AT_ARGS grid, stream, (const bf16_t*)q, ldq, out, ldo, (const bf16_t*)kcache, (const bf16_t*)vcache, block_table, max_blocks, \
                 tiles, positions, maps, per_kv, kv_heads * maps, kv_heads, dv, page_shift, window, scale, softcap, partial, per_split, \
-                share, q_slots, keep_first, sinks
+                share, q_slots, keep_first, sinks, chunk, slopes
 #define AT_DB(N)                                  \
   switch (db) {                                   \
     case 1: rc = launch_tiles<N, 1>(AT_ARGS); break; \

@@ -22,6 +22,7 @@
 #include <math.h>
 
 #include "common.h"
+#include "recurrence.h"
 
 #define CONV_MAX_TAPS 16
 #define GDR_COLS 16    // value columns of a workgroup (4 per wave)
@@ -54,34 +55,6 @@ __global__ __launch_bounds__(256) void short_conv_silu_kernel(const T* __restric
     acc = fmaf(ldf(w, (size_t)c * taps + (taps - 1 - j)), v, acc);
   }
   stf(y + (size_t)t * ldy, c, silu_f(acc + shift));
-}
-
-// first row and number of rows of request `req` in the ascending list row_req[0 .. n)
-__device__ __forceinline__ void rows_of_request(const int* __restrict__ row_req, int n, int req, int& lo, int& cnt) {
-  if (req < n) {
-    // a step of single rows has request r's one row at place r: three loads side by side in place of two searches.
-    // In an ascending list, a place that holds r between two neighbours that do not is all of r's rows.
-    const int here = row_req[req];
-    const int before = req > 0 ? row_req[req - 1] : -1;
-    const int after = req + 1 < n ? row_req[req + 1] : 0x7fffffff;
-    if (here == req && before != req && after != req) {
-      lo = req;
-      cnt = 1;
-      return;
-    }
-  }
-  int a = 0, b = n;
-  while (a < b) {
-    const int mid = (a + b) >> 1;
-    if (row_req[mid] < req) a = mid + 1; else b = mid;
-  }
-  lo = a;
-  b = n;
-  while (a < b) {
-    const int mid = (a + b) >> 1;
-    if (row_req[mid] <= req) a = mid + 1; else b = mid;
-  }
-  cnt = a - lo;
 }
 
 template <typename T>
@@ -195,14 +168,6 @@ struct GdrArgs {
   const int* state_slots;
   int n_rows, heads, kv_heads, dk, dv;
 };
-
-__device__ __forceinline__ float row16_sum(float d) {  // over a row of 16 lanes, left in all of them
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0xB1, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x4E, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x141, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x140, 0xF, 0xF, true));
-  return d;
-}
 
 // thread = wave * 64 + c * 16 + part: column blockIdx.z * 16 + wave * 4 + c, key rows part * E .. + E
 // CHANNEL: the decay is a vector over the key channels (S's rows) instead of one number per head:

@@ -1,0 +1,522 @@
+// Linear attention with a fixed decay per head: S <- d_h S + k v^T, o = S^T q with S [dk, dv] per head, no softmax and no
+// denominator. fp32 or bf16 projections, everything from there on and the state in fp32. q, k and v are columns of one
+// projection's rows; on their way in they pass, as asked, silu (all three), a rotation of the pairs (i, i + rot / 2) among
+// the first rot entries of every q and k head by the row's position, and a constant on k. A request's rows of a step are
+// consecutive and in order (row_req ascends), their positions too.
+//
+//   linear_scan     token by token, for steps of few rows per request and for sizes that the chunked form does not take:
+//                   a workgroup of four waves owns 16 value columns of one head of one request, 16 lanes per column with
+//                   a sixteenth of the state rows each; the state stays in registers while the rows are walked.
+//   linear_states   the chunked form, for portions of prompts: with the decay fixed, C tokens move the state by
+//                   S' = d^C S + sum_t d^(C - 1 - t) k_t v_t^T, one product of a [dk, C] and a [C, dv] matrix. One
+//                   workgroup per (request, head, 16 value columns) walks the request's chunks of 64 rows in order and
+//                   leaves the state in front of every chunk in a scratch array; the last one is the request's new state.
+//   linear_outputs  the rest is independent per chunk and head: o_t = d^(t + 1) S^T q_t + sum_(s <= t) d^(t - s) (q_t .
+//                   k_s) v_s, three matrix products.
+//   The products of the chunked form are fp32 matrix-core instructions (v_mfma_f32_16x16x4_f32: fp32 operands, fp32
+//   sums), so the two forms differ by the order of their sums only. The powers of a head's decay come from a table
+//   [heads, 65] that the host computes in double.
+//
+// State of one request: [heads, dv, dk] (a head's matrix column by column).
+#include <math.h>
+
+#include "common.h"
+#include "recurrence.h"
+
+#define LIN_COLS 16
+#define LIN_PARTS 16
+#define LIN_ROWS 64            // rows of a chunk
+#define LIN_POWERS (LIN_ROWS + 1)
+
+typedef float floatx4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ floatx4 mfma_f32(float a, float b, floatx4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+struct LinArgs {
+  const void* y;      // [rows, ld]: q (heads x dk) from q_off, k (heads x dk) from k_off, v (heads x dv) from v_off
+  int ld, q_off, k_off, v_off;
+  const int* positions;
+  const float* cos_t;  // [positions, rot / 2]
+  const float* sin_t;
+  int rot, silu;
+  float k_scale;
+  const float* powers;  // [heads, 65]: d^0 .. d^64
+  float* state;         // [slots, heads, dv, dk]
+  float* out;           // [rows, ldo]: heads x dv
+  int ldo;
+  const int* row_req;
+  const int* state_slots;
+  int n_rows, heads, dk, dv;
+  // the chunked form
+  const int* requests;  // [requests, 3]: first row, rows, first chunk
+  const int* chunks;    // [chunks, 2]: first row, rows
+  float* before;        // [chunks, heads, dv, dk]: the state in front of every chunk
+};
+
+__device__ __forceinline__ float lin_act(float z, int silu) { return silu ? z / (1.0f + expf(-z)) : z; }
+
+// thread = cw * 16 + part: column blockIdx.z * 16 + cw, state rows part * E .. + E. C: rows staged at a time
+template <typename T, int E, int C, bool ROT>
+__global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
+  constexpr int NP = LIN_PARTS * E;          // the key size, padded with zeros
+  constexpr int ROWF = 2 * NP + LIN_COLS + 4;  // q | k | v of the workgroup's columns | -
+  constexpr int NQK = (C * 2 * NP + 255) / 256;
+  __shared__ __align__(16) float sm[C * ROWF];
+  const int tid = threadIdx.x;
+  const int part = tid & 15, cw = tid >> 4;
+  const int req = blockIdx.x, h = blockIdx.y;
+  const int col0 = blockIdx.z * LIN_COLS;
+  const int col = col0 + cw;
+  const bool col_on = col < A.dv;
+  int lo, n;
+  rows_of_request(A.row_req, A.n_rows, req, lo, n);
+  if (n == 0) return;
+  const int dk = A.dk;
+  const int i0 = part * E;
+  float* S_at = A.state + ((size_t)A.state_slots[req] * A.heads + h) * dk * A.dv;
+  float S[E];
+  // every lane loads from a place that exists and drops what it does not own, so that the loads are in flight together
+  const bool wide = E >= 4 && (dk & 3) == 0;  // then a lane's entries start on 16 bytes and end with the column
+  if (wide) {
+#pragma unroll
+    for (int e = 0; e < E; e += 4) {
+      const bool own = col_on && i0 + e < dk;
+      const float4 s = *reinterpret_cast<const float4*>(S_at + (own ? (size_t)col * dk + i0 + e : 0));
+      S[e] = own ? s.x : 0.f;
+      S[(e + 1) % E] = own ? s.y : 0.f;
+      S[(e + 2) % E] = own ? s.z : 0.f;
+      S[(e + 3) % E] = own ? s.w : 0.f;
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const bool own = col_on && i0 + e < dk;
+      const float s = S_at[own ? (size_t)col * dk + i0 + e : 0];
+      S[e] = own ? s : 0.f;
+    }
+  }
+  const T* y = (const T*)A.y;
+  const int half = A.rot >> 1;
+  const int pos0 = ROT ? A.positions[lo] : 0;
+  const float d = A.powers[(size_t)h * LIN_POWERS + 1];
+  const size_t q_at = (size_t)A.q_off + (size_t)h * dk, k_at = (size_t)A.k_off + (size_t)h * dk;
+  const size_t v_at = (size_t)A.v_off + (size_t)h * A.dv + col0;
+  for (int r0 = 0; r0 < n; r0 += C) {
+    const int have = min(C, n - r0);
+    if (r0) __syncthreads();  // the rows before have been read
+#pragma unroll
+    for (int j = 0; j < NQK; ++j) {
+      const int idx = tid + 256 * j;
+      if (C * 2 * NP % 256 && idx >= C * 2 * NP) break;
+      const int t = idx / (2 * NP), w = idx % (2 * NP);
+      const int i = w % NP;
+      const bool own = t < have && i < dk;
+      const T* row = y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + (w < NP ? q_at : k_at);
+      float p = lin_act(ldf(row, own ? i : 0), A.silu);
+      if (ROT) {
+        const bool turns = own && i < A.rot;
+        const int f = turns ? (i < half ? i : i - half) : 0;
+        const float o = lin_act(ldf(row, turns ? (i < half ? i + half : i - half) : 0), A.silu);
+        const size_t at = (size_t)(pos0 + r0 + (own ? t : 0)) * half + f;
+        const float c = A.cos_t[at], s = A.sin_t[at];
+        if (turns) p = i < half ? p * c - o * s : p * c + o * s;
+      }
+      if (w >= NP) p *= A.k_scale;
+      sm[t * ROWF + w] = own ? p : 0.f;
+    }
+    if (tid < C * LIN_COLS) {
+      const int t = tid / LIN_COLS, cc = tid % LIN_COLS;
+      const bool own = t < have && col0 + cc < A.dv;
+      const float p = lin_act(ldf(y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + v_at, own ? cc : 0), A.silu);
+      sm[t * ROWF + 2 * NP + cc] = own ? p : 0.f;
+    }
+    __syncthreads();
+    for (int t = 0; t < have; ++t) {
+      const float* row = sm + t * ROWF;
+      const float v = row[2 * NP + cw];
+      float o = 0.f;
+#pragma unroll
+      for (int e = 0; e < E; ++e) {
+        S[e] = fmaf(v, row[NP + i0 + e], d * S[e]);
+        o = fmaf(S[e], row[i0 + e], o);
+      }
+      o = row16_sum(o);
+      if (part == 0 && col_on) A.out[(size_t)(lo + r0 + t) * A.ldo + (size_t)h * A.dv + col] = o;
+    }
+  }
+  if (wide) {
+#pragma unroll
+    for (int e = 0; e < E; e += 4)
+      if (col_on && i0 + e < dk)
+        *reinterpret_cast<float4*>(S_at + (size_t)col * dk + i0 + e) = make_float4(S[e], S[(e + 1) % E], S[(e + 2) % E], S[(e + 3) % E]);
+  } else {
+#pragma unroll
+    for (int e = 0; e < E; ++e)
+      if (col_on && i0 + e < dk) S_at[(size_t)col * dk + i0 + e] = S[e];
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------
+// the chunked form: dk and dv in multiples of 16 up to 256, rot in multiples of 8, rows and offsets on 4 elements
+
+template <typename T>
+struct Raw4;  // four neighbouring elements as they lie in memory
+template <>
+struct Raw4<float> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* p) { v = *(const float4*)p; }
+  __device__ __forceinline__ float get(int e) const { return e == 0 ? v.x : e == 1 ? v.y : e == 2 ? v.z : v.w; }
+};
+template <>
+struct Raw4<bf16_t> {
+  uint2 v;
+  __device__ __forceinline__ void load(const bf16_t* p) { v = *(const uint2*)p; }
+  __device__ __forceinline__ float get(int e) const {
+    const uint32_t w = e < 2 ? v.x : v.y;
+    return __uint_as_float((e & 1) ? (w & 0xffff0000u) : (w << 16));
+  }
+};
+
+// Two groups of four entries of a q or k head that the same thread brings in: entries i1 .. + 4 and i2 .. + 4. Below rot / 2
+// they are the two sides of four turned pairs, beyond it neighbours that pass unturned.
+template <typename T, bool ROT>
+struct HeadUnit {
+  Raw4<T> a, b;
+  float4 c, s;
+  int i1, i2;
+  bool turns;
+  __device__ __forceinline__ void load(const T* head, int u, int rot, const float* cos_row, const float* sin_row) {
+    const int half = rot >> 1;
+    turns = ROT && u * 4 < half;
+    i1 = turns ? u * 4 : rot + 2 * (u * 4 - half);
+    i2 = turns ? i1 + half : i1 + 4;
+    a.load(head + i1);
+    b.load(head + i2);
+    if (ROT) {
+      const int f = turns ? u * 4 : 0;
+      c = *(const float4*)(cos_row + f);
+      s = *(const float4*)(sin_row + f);
+    }
+  }
+  __device__ __forceinline__ void store(float* row, bool on, int silu, float mul) const {
+    float p[4], q[4];
+    const float cc[4] = {c.x, c.y, c.z, c.w}, ss[4] = {s.x, s.y, s.z, s.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      p[e] = lin_act(a.get(e), silu);
+      q[e] = lin_act(b.get(e), silu);
+      if (ROT && turns) {
+        const float u = p[e], v = q[e];
+        p[e] = u * cc[e] - v * ss[e];
+        q[e] = v * cc[e] + u * ss[e];
+      }
+      p[e] = on ? p[e] * mul : 0.f;
+      q[e] = on ? q[e] * mul : 0.f;
+    }
+    *(float4*)(row + i1) = float4{p[0], p[1], p[2], p[3]};
+    *(float4*)(row + i2) = float4{q[0], q[1], q[2], q[3]};
+  }
+};
+
+// grid (request, head, 16 value columns), four waves. Wave w accumulates the state rows of its DT tiles of 16; lane l of
+// a tile holds rows 4 (l / 16) .. + 4 of column l % 16.
+template <typename T, int DT, bool ROT>
+__global__ __launch_bounds__(256) void linear_states_kernel(LinArgs A) {
+  constexpr int DKP = DT * 64;
+  constexpr int KLD = DKP + 16;   // four neighbouring rows of 16 entries lie in different banks
+  constexpr int NU = DKP / 8 * LIN_ROWS / 256;
+  __shared__ __align__(16) float Ks[LIN_ROWS * KLD];
+  __shared__ __align__(16) float Vs[LIN_ROWS * LIN_COLS];
+  const int tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
+  const int req = blockIdx.x, h = blockIdx.y, col = blockIdx.z * LIN_COLS + l16;
+  const int lo = A.requests[req * 3], n = A.requests[req * 3 + 1], chunk0 = A.requests[req * 3 + 2];
+  const int dk = A.dk, dv = A.dv, units = dk >> 3;
+  if (n <= 0) return;
+  const float* pw = A.powers + (size_t)h * LIN_POWERS;
+  const T* y = (const T*)A.y;
+  const T* kh = y + A.k_off + (size_t)h * dk;
+  const T* vh = y + A.v_off + (size_t)h * dv + blockIdx.z * LIN_COLS;
+  const int pos0 = ROT ? A.positions[lo] : 0;
+  const int half = A.rot >> 1;
+  float* S_at = A.state + (((size_t)A.state_slots[req] * A.heads + h) * dv + col) * dk;
+  floatx4 S[DT];
+#pragma unroll
+  for (int j = 0; j < DT; ++j) {
+    const int i = (wave * DT + j) * 16 + 4 * g;
+    S[j] = i < dk ? *(const floatx4*)(S_at + i) : floatx4{0.f, 0.f, 0.f, 0.f};
+  }
+  HeadUnit<T, ROT> ku[NU];
+  Raw4<T> vu;
+  auto request = [&](int r0) {  // rows beyond the request's last are read from its last
+    const int last = n - 1;
+#pragma unroll
+    for (int j = 0; j < NU; ++j) {
+      const int idx = tid + 256 * j;
+      const int t = min(r0 + idx / (DKP / 8), last), u = min(idx % (DKP / 8), units - 1);
+      ku[j].load(kh + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
+                 ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
+    }
+    vu.load(vh + (size_t)(lo + min(r0 + (tid >> 2), last)) * A.ld + (tid & 3) * 4);
+  };
+  request(0);
+  for (int r0 = 0, c = chunk0; r0 < n; r0 += LIN_ROWS, ++c) {
+    const int have = min(LIN_ROWS, n - r0);
+    if (r0) __syncthreads();  // the chunk before has been read
+#pragma unroll
+    for (int j = 0; j < NU; ++j) {
+      const int idx = tid + 256 * j;
+      const int t = idx / (DKP / 8), u = idx % (DKP / 8);
+      float* row = Ks + t * KLD;
+      if (u < units) {
+        ku[j].store(row, t < have, A.silu, A.k_scale);
+      } else {  // the padding behind the key size
+        *(float4*)(row + u * 8) = float4{0.f, 0.f, 0.f, 0.f};
+        *(float4*)(row + u * 8 + 4) = float4{0.f, 0.f, 0.f, 0.f};
+      }
+    }
+    {
+      const int t = tid >> 2;
+      const float w = t < have ? pw[max(have - 1 - t, 0)] : 0.f;
+      float v[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act(vu.get(e), A.silu) * w : 0.f;
+      *(float4*)(Vs + t * LIN_COLS + (tid & 3) * 4) = float4{v[0], v[1], v[2], v[3]};
+    }
+    __syncthreads();
+    if (r0 + LIN_ROWS < n) request(r0 + LIN_ROWS);  // in flight while this chunk is worked through
+    float* S_c = A.before + (((size_t)c * A.heads + h) * dv + col) * dk;
+    const float dC = pw[have];
+#pragma unroll
+    for (int j = 0; j < DT; ++j) {
+      const int i = (wave * DT + j) * 16 + 4 * g;
+      if (i < dk) *(floatx4*)(S_c + i) = S[j];
+      S[j] *= dC;
+    }
+#pragma unroll 4
+    for (int t0 = 0; t0 < LIN_ROWS; t0 += 4) {
+      const float b = Vs[(t0 + g) * LIN_COLS + l16];
+#pragma unroll
+      for (int j = 0; j < DT; ++j) S[j] = mfma_f32(Ks[(t0 + g) * KLD + (wave * DT + j) * 16 + l16], b, S[j]);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < DT; ++j) {
+    const int i = (wave * DT + j) * 16 + 4 * g;
+    if (i < dk) *(floatx4*)(S_at + i) = S[j];
+  }
+}
+
+// grid (chunk, head), eight waves. LDS: Q [64][dk], K [64][dk] (later V [64][dv] in its place), P [64][64].
+template <typename T, int DT, bool ROT>
+__global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
+  constexpr int DKP = DT * 64;
+  constexpr int QLD = DKP + 4;
+  constexpr int PLD = LIN_ROWS + 4;
+  constexpr int UN = DKP / 8;
+  constexpr int NU = UN * LIN_ROWS / 512;
+  extern __shared__ __align__(16) float lin_smem[];
+  float* Qs = lin_smem;
+  float* Ps = Qs + LIN_ROWS * QLD;
+  float* Ks = Ps + LIN_ROWS * PLD;
+  const int tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
+  const int c = blockIdx.x, h = blockIdx.y;
+  const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
+  const int dk = A.dk, dv = A.dv, units = dk >> 3, vld = dv + 4;
+  const float* pw = A.powers + (size_t)h * LIN_POWERS;
+  const T* y = (const T*)A.y;
+  const int pos0 = ROT ? A.positions[lo] : 0;
+  const int half = A.rot >> 1;
+#pragma unroll
+  for (int which = 0; which < 2; ++which) {
+    const T* head = y + (which ? A.k_off : A.q_off) + (size_t)h * dk;
+    HeadUnit<T, ROT> hu[NU];
+#pragma unroll
+    for (int j = 0; j < NU; ++j) {
+      const int idx = tid + 512 * j;
+      const int t = min(idx / UN, have - 1), u = min(idx % UN, units - 1);
+      hu[j].load(head + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
+                 ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
+    }
+#pragma unroll
+    for (int j = 0; j < NU; ++j) {
+      const int idx = tid + 512 * j;
+      const int t = idx / UN, u = idx % UN;
+      if (u < units) hu[j].store((which ? Ks : Qs) + t * QLD, t < have, A.silu, which ? A.k_scale : 1.0f);
+    }
+  }
+  __syncthreads();
+  // P[i][j] = d^(i - j) (q_i . k_j) for j <= i: ten tiles of 16 x 16
+  for (int tile = wave; tile < 10; tile += 8) {
+    const int rt = tile >= 6 ? 3 : tile >= 3 ? 2 : tile >= 1 ? 1 : 0;
+    const int ct = tile - rt * (rt + 1) / 2;
+    const float* qa = Qs + (rt * 16 + l16) * QLD + 4 * g;
+    const float* kb = Ks + (ct * 16 + l16) * QLD + 4 * g;
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k0 = 0; k0 < dk; k0 += 16) {
+      const floatx4 a = *(const floatx4*)(qa + k0), b = *(const floatx4*)(kb + k0);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc = mfma_f32(a[e], b[e], acc);
+    }
+    const int j = ct * 16 + l16;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = rt * 16 + 4 * g + e;
+      Ps[i * PLD + j] = j <= i ? acc[e] * pw[i - j] : 0.f;
+    }
+  }
+  __syncthreads();  // K has been read: V takes its place
+  for (int idx = tid; idx < LIN_ROWS * (dv >> 2); idx += 512) {
+    const int t = idx / (dv >> 2), e4 = idx % (dv >> 2) * 4;
+    Raw4<T> r;
+    r.load(y + (size_t)(lo + min(t, have - 1)) * A.ld + A.v_off + (size_t)h * dv + e4);
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act(r.get(e), A.silu) : 0.f;
+    *(float4*)(Ks + t * vld + e4) = float4{v[0], v[1], v[2], v[3]};
+  }
+  __syncthreads();
+  // a wave takes two row tiles (one early, one late: their causal parts add up to the same) of a tile of value columns
+  const int rts[2] = {wave & 1, 3 - (wave & 1)};
+  for (int ct = wave >> 1; ct * 16 < dv; ct += 4) {
+    const float* S_c = A.before + (((size_t)c * A.heads + h) * dv + ct * 16 + l16) * dk + 4 * g;
+    floatx4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll 4
+    for (int k0 = 0; k0 < dk; k0 += 16) {
+      const floatx4 b = *(const floatx4*)(S_c + k0);
+#pragma unroll
+      for (int r = 0; r < 2; ++r) {
+        const floatx4 a = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], b[e], acc[r]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 2; ++r) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc[r][e] *= pw[rts[r] * 16 + 4 * g + e + 1];
+      const float* pa = Ps + (rts[r] * 16 + l16) * PLD + 4 * g;
+      for (int j0 = 0; j0 < (rts[r] + 1) * 16; j0 += 16) {
+        const floatx4 a = *(const floatx4*)(pa + j0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], Ks[(j0 + 4 * g + e) * vld + ct * 16 + l16], acc[r]);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = rts[r] * 16 + 4 * g + e;
+        if (t < have) A.out[(size_t)(lo + t) * A.ldo + (size_t)h * dv + ct * 16 + l16] = acc[r][e];
+      }
+    }
+  }
+}
+
+template <typename T, int DT, bool ROT>
+static int launch_outputs(dim3 grid, hipStream_t stream, const LinArgs& A) {
+  const int qld = DT * 64 + 4, vld = A.dv + 4;
+  const size_t smem = (size_t)LIN_ROWS * (qld + (LIN_ROWS + 4) + (qld > vld ? qld : vld)) * sizeof(float);
+  static size_t raised = 64 * 1024;
+  if (smem > raised) {
+    if (smem > 160 * 1024 ||
+        hipFuncSetAttribute((const void*)linear_outputs_kernel<T, DT, ROT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess)
+      return -1;
+    raised = 160 * 1024;
+  }
+  linear_outputs_kernel<T, DT, ROT><<<grid, 512, smem, stream>>>(A);
+  return 0;
+}
+
+static int check_args(const char* name, const LinArgs& A, int n_requests) {
+  if (A.heads <= 0 || A.heads > 65535 || A.dk <= 0 || A.dk > LIN_PARTS * 16 || A.dv <= 0 || A.dv > LIN_COLS * 65535)
+    JLLM_FAIL("%s: %d heads, key size %d (1..%d are taken), value size %d", name, A.heads, A.dk, LIN_PARTS * 16, A.dv);
+  if (n_requests <= 0 || n_requests > A.n_rows) JLLM_FAIL("%s: %d requests in %d rows", name, n_requests, A.n_rows);
+  if (A.q_off < 0 || A.k_off < 0 || A.v_off < 0 || A.ld < A.q_off + A.heads * A.dk || A.ld < A.k_off + A.heads * A.dk ||
+      A.ld < A.v_off + A.heads * A.dv || A.ldo < A.heads * A.dv)
+    JLLM_FAIL("%s: short rows", name);
+  if (A.rot < 0 || A.rot % 2 || A.rot > A.dk || (A.rot && (!A.cos_t || !A.sin_t || !A.positions)))
+    JLLM_FAIL("%s: a rotary width of %d for heads of %d", name, A.rot, A.dk);
+  return 0;
+}
+
+extern "C" int jllm_linear_scan(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
+                                const float* cos_t, const float* sin_t, int rot, int silu, float k_scale, const float* powers,
+                                float* state, float* out, int ldo, const int* row_req, const int* state_slots, int n_rows,
+                                int n_requests, int heads, int dk, int dv, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, row_req, state_slots,
+            n_rows, heads, dk, dv, nullptr, nullptr, nullptr};
+  if (check_args("linear_scan", A, n_requests) != 0) return -1;
+  dim3 grid(n_requests, heads, (dv + LIN_COLS - 1) / LIN_COLS);
+  const int per_lane = (dk + LIN_PARTS - 1) / LIN_PARTS;
+  const bool few = n_rows <= 2 * n_requests;
+#define LIN_LAUNCH(E)                                                             \
+  do {                                                                            \
+    if (few && rot)                                                               \
+      linear_scan_kernel<T, E, 2, true><<<grid, 256, 0, stream>>>(A);             \
+    else if (few)                                                                 \
+      linear_scan_kernel<T, E, 2, false><<<grid, 256, 0, stream>>>(A);            \
+    else if (rot)                                                                 \
+      linear_scan_kernel<T, E, 16, true><<<grid, 256, 0, stream>>>(A);            \
+    else                                                                          \
+      linear_scan_kernel<T, E, 16, false><<<grid, 256, 0, stream>>>(A);           \
+  } while (0)
+  JLLM_DISPATCH_1(dtype, T, {
+    if (per_lane <= 2)
+      LIN_LAUNCH(2);
+    else if (per_lane <= 4)
+      LIN_LAUNCH(4);
+    else if (per_lane <= 8)
+      LIN_LAUNCH(8);
+    else
+      LIN_LAUNCH(16);
+  })
+#undef LIN_LAUNCH
+  JLLM_CHECK_LAUNCH("linear_scan");
+  return 0;
+}
+
+// Returns 1 (declined) for sizes that the chunked form does not take. requests [n_requests, 3]: first row, rows, first
+// chunk; chunks [n_chunks, 2]: first row, rows (at most 64, of one request, in order); before: fp32 [n_chunks, heads, dv, dk]
+extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
+                                  const float* cos_t, const float* sin_t, int rot, int silu, float k_scale,
+                                  const float* powers, float* state, float* out, int ldo, const int* requests,
+                                  const int* chunks, int n_chunks, float* before, const int* state_slots, int n_rows,
+                                  int n_requests, int heads, int dk, int dv, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, nullptr, state_slots,
+            n_rows, heads, dk, dv, requests, chunks, before};
+  if (check_args("linear_chunks", A, n_requests) != 0) return -1;
+  if (n_chunks < n_requests || n_chunks > n_rows || !requests || !chunks || !before) JLLM_FAIL("linear_chunks: %d chunks of %d rows of %d requests", n_chunks, n_rows, n_requests);
+  const size_t bytes4 = dtype == JLLM_F32 ? 16 : 8;
+  if ((dk & 15) || (dv & 15) || dk > 256 || dv > 256 || (rot & 7)) return 1;
+  if ((ld & 3) || (q_off & 3) || (k_off & 3) || (v_off & 3) || ((uintptr_t)y % bytes4) || ((uintptr_t)state & 15) || ((uintptr_t)before & 15) ||
+      (rot && (((uintptr_t)cos_t & 15) || ((uintptr_t)sin_t & 15))))
+    return 1;
+  const dim3 sgrid(n_requests, heads, dv / LIN_COLS), ogrid(n_chunks, heads);
+  int rc = 0;
+#define LIN_CHUNKS(DT)                                                                     \
+  do {                                                                                     \
+    if (rot) {                                                                             \
+      linear_states_kernel<T, DT, true><<<sgrid, 256, 0, stream>>>(A);                     \
+      rc = launch_outputs<T, DT, true>(ogrid, stream, A);                                  \
+    } else {                                                                               \
+      linear_states_kernel<T, DT, false><<<sgrid, 256, 0, stream>>>(A);                    \
+      rc = launch_outputs<T, DT, false>(ogrid, stream, A);                                 \
+    }                                                                                      \
+  } while (0)
+  JLLM_DISPATCH_1(dtype, T, {
+    if (dk <= 64)
+      LIN_CHUNKS(1);
+    else if (dk <= 128)
+      LIN_CHUNKS(2);
+    else
+      LIN_CHUNKS(4);
+  })
+#undef LIN_CHUNKS
+  if (rc < 0) JLLM_FAIL("linear_chunks: cannot reserve LDS");
+  JLLM_CHECK_LAUNCH("linear_chunks");
+  return 0;
+}

@@ -13,11 +13,13 @@
 //                     arithmetic is one sequence of operations whatever the cut of the prompt (the tokens of a full
 //                     chunk are only interleaved, their sums over the lanes taken together), so fp32 results do not
 //                     depend on it.
-//   gated_group_norm  out = rmsnorm_g(y * silu(z)) * w: the gate comes first, then every one of `groups` equal parts
-//                     of a row is divided by its own root mean square
+//   gated_group_norm  out = rmsnorm_g(y * gate(z)) * w: the gate (silu or sigmoid) comes first, then every one of
+//                     `groups` equal parts of a row is divided by its own root mean square; or, with `gate_last`,
+//                     out = rmsnorm_g(y) * w * gate(z)
 #include <math.h>
 
 #include "common.h"
+#include "recurrence.h"
 
 #define SSM_COLS 16
 #define SSM_PARTS 16
@@ -39,41 +41,6 @@ struct SsmArgs {
   int n_rows, heads, groups, n, dv;
 };
 
-__device__ __forceinline__ void ssm_rows_of_request(const int* __restrict__ row_req, int n, int req, int& lo, int& cnt) {
-  if (req < n) {
-    // a step of single rows has request r's one row at place r: three loads side by side in place of two searches.
-    // In an ascending list, a place that holds r between two neighbours that do not is all of r's rows.
-    const int here = row_req[req];
-    const int before = req > 0 ? row_req[req - 1] : -1;
-    const int after = req + 1 < n ? row_req[req + 1] : 0x7fffffff;
-    if (here == req && before != req && after != req) {
-      lo = req;
-      cnt = 1;
-      return;
-    }
-  }
-  int a = 0, b = n;
-  while (a < b) {
-    const int mid = (a + b) >> 1;
-    if (row_req[mid] < req) a = mid + 1; else b = mid;
-  }
-  lo = a;
-  b = n;
-  while (a < b) {
-    const int mid = (a + b) >> 1;
-    if (row_req[mid] <= req) a = mid + 1; else b = mid;
-  }
-  cnt = a - lo;
-}
-
-__device__ __forceinline__ float ssm_row16_sum(float d) {  // over a row of 16 lanes, left in all of them
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0xB1, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x4E, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x141, 0xF, 0xF, true));
-  d += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, d), 0x140, 0xF, 0xF, true));
-  return d;
-}
-
 // thread = cw * 16 + part: column blockIdx.z * 16 + cw, state rows part * E .. + E
 // FEW: the form for steps of few rows per request (decoding). It leaves out the interleaved walk over a full chunk, whose
 // registers would halve the workgroups that a compute unit holds: such a step is a wait for each request's state, and
@@ -92,7 +59,7 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs A) {
   const int col = col0 + cw;
   const bool col_on = col < A.dv;
   int lo, n;
-  ssm_rows_of_request(A.row_req, A.n_rows, req, lo, n);
+  rows_of_request(A.row_req, A.n_rows, req, lo, n);
   if (n == 0) return;
   const int ns = A.n;
   const int grp = h / (A.heads / A.groups);
@@ -192,14 +159,14 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs A) {
 #pragma unroll
       for (int t = 0; t < C; ++t) yp[t] = token(t);
 #pragma unroll
-      for (int t = 0; t < C; ++t) yp[t] = ssm_row16_sum(yp[t]);
+      for (int t = 0; t < C; ++t) yp[t] = row16_sum(yp[t]);
       float mine = yp[0];  // lane `part` of a column writes token `part`
 #pragma unroll
       for (int t = 1; t < C; ++t) mine = part == t ? yp[t] : mine;
       if (col_on) A.out[(size_t)(lo + r0 + part) * A.ldo + (size_t)h * A.dv + col] = fmaf(skip, sm[part * ROWF + 2 * NP + cw], mine);
     } else {
       for (int t = 0; t < have; ++t) {
-        const float y = ssm_row16_sum(token(t));
+        const float y = row16_sum(token(t));
         if (part == 0 && col_on) A.out[(size_t)(lo + r0 + t) * A.ldo + (size_t)h * A.dv + col] = fmaf(skip, sm[t * ROWF + 2 * NP + cw], y);
       }
     }
@@ -254,41 +221,46 @@ extern "C" int jllm_ssm_scan(const void* xbc, int ld, const void* dt, int ldt, i
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
-// one workgroup per (row, group): t = y * silu(z) over the group's entries, out = t / sqrt(mean(t^2) + eps) * w
+// one workgroup per (row, group): t = y * gate(z) over the group's entries, out = t / sqrt(mean(t^2) + eps) * w, or with
+// `gate_last` t = y and the gate multiplies the result
+__device__ __forceinline__ float group_gate(float z, int fn) { return (fn == 1 ? z : 1.0f) / (1.0f + expf(-z)); }
+
 template <typename TZ, typename TW, typename TO>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ y, int ldy, const TZ* __restrict__ z,
                                                                int ldz, const TW* __restrict__ w, float eps, int per,
-                                                               TO* __restrict__ out, int ldo) {
+                                                               TO* __restrict__ out, int ldo, int gate_fn, int gate_last,
+                                                               float out_mul) {
   __shared__ float red[4];
   const int r = blockIdx.x, g = blockIdx.y;
   const float* yr = y + (size_t)r * ldy + (size_t)g * per;
   const TZ* zr = z + (size_t)r * ldz + (size_t)g * per;
   float ss = 0.f;
   for (int i = threadIdx.x; i < per; i += 256) {
-    const float zz = ldf(zr, i);
-    const float t = yr[i] * (zz / (1.0f + expf(-zz)));
+    const float t = gate_last ? yr[i] : yr[i] * group_gate(ldf(zr, i), gate_fn);
     ss = fmaf(t, t, ss);
   }
   ss = block_sum<4>(ss, red);
   const float s = norm_scale(ss, per, eps);
   for (int i = threadIdx.x; i < per; i += 256) {
-    const float zz = ldf(zr, i);
-    const float t = yr[i] * (zz / (1.0f + expf(-zz)));
-    stf(out + (size_t)r * ldo, (size_t)g * per + i, (t * s) * ldf(w, (size_t)g * per + i));
+    const float gate = group_gate(ldf(zr, i), gate_fn), wi = ldf(w, (size_t)g * per + i);
+    const float v = gate_last ? yr[i] * s * wi * gate : yr[i] * gate * s * wi;
+    stf(out + (size_t)r * ldo, (size_t)g * per + i, v * out_mul);
   }
 }
 
+// gate_fn: 0 sigmoid, 1 silu
 extern "C" int jllm_gated_group_norm(const float* y, int ldy, const void* z, int ldz, int z_dtype, const void* w, int w_dtype,
                                      float eps, int n_rows, int width, int groups, void* out, int out_dtype, int ldo,
-                                     hipStream_t stream) {
+                                     int gate_fn, int gate_last, float out_mul, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (width <= 0 || groups <= 0 || width % groups || groups > 65535) JLLM_FAIL("gated_group_norm: rows of %d in %d groups", width, groups);
   if (ldy < width || ldz < width || ldo < width) JLLM_FAIL("gated_group_norm: short rows");
+  if (gate_fn != 0 && gate_fn != 1) JLLM_FAIL("gated_group_norm: gate function %d (0 sigmoid and 1 silu are built)", gate_fn);
   JLLM_DISPATCH_1(z_dtype, TZ, {
     JLLM_DISPATCH_1(w_dtype, TW, {
       JLLM_DISPATCH_1(out_dtype, TO, {
-        gated_group_norm_kernel<TZ, TW, TO><<<dim3(n_rows, groups), 256, 0, stream>>>(y, ldy, (const TZ*)z, ldz, (const TW*)w, eps,
-                                                                                     width / groups, (TO*)out, ldo);
+        gated_group_norm_kernel<TZ, TW, TO><<<dim3(n_rows, groups), 256, 0, stream>>>(
+            y, ldy, (const TZ*)z, ldz, (const TW*)w, eps, width / groups, (TO*)out, ldo, gate_fn, gate_last, out_mul);
       })
     })
   })

@@ -80,11 +80,15 @@ def _declare(lib) -> None:
         "jllm_streams_write": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P],
         "jllm_concat_rows": [_P, _P, _I, _I, _P, _I, _I, _P],
         "jllm_ssm_scan": [_P, _I, _P, _I, _I, _I, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P],
-        "jllm_gated_group_norm": [_P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P, _I, _I, _P],
+        "jllm_gated_group_norm": [_P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P, _I, _I, _I, _I, _F, _P],
+        "jllm_linear_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
+        "jllm_linear_chunks": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
+        "jllm_rms_seam": [_P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _P, _F, _P, _F, _P, _I, _I, _P, _P, _P, _P],
+        "jllm_token_shift": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
         "jllm_copy_page_rows": [_P, _I, _I, _I, _I, _L, _I, _I, _I, _P],
         "jllm_layernorm_seam": [_P, _P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _P, _P, _P, _P, _I, _F, _P, _I, _I, _P],
-        "jllm_qkv_prepare": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _F, _P, _P, _I, _F, _I, _P, _P, _I, _I, _I, _P],
-        "jllm_attention_dv_generic": [_P, _I, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _P],
+        "jllm_qkv_prepare": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _F, _P, _P, _I, _F, _I, _P, _P, _I, _I, _I, _P, _I, _I, _P],
+        "jllm_attention_dv_generic": [_P, _I, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _I, _P, _P],
         "jllm_heads_finish": [_P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P, _I, _P, _I, _I, _I, _F, _P, _I, _I, _I, _P],
         "jllm_heads_finish_split": [_P, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P, _I, _P, _I, _I, _I, _F, _P, _I, _I, _I, _P, _P],
         "jllm_short_conv": [_P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _P, _P],
@@ -121,7 +125,7 @@ _OPTIONAL_SIGS = {
     "jllm_latent_attention_bf16": [_P, _I, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _P, _P],
     "jllm_latent_heads_bf16": [_P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P],
     "jllm_gemm_mfma_grouped_bf16": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _P, _I, _P],
-    "jllm_attention_dv_bf16": [_P, _I, _P, _I, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P, _I, _I, _I, _P, _P],
+    "jllm_attention_dv_bf16": [_P, _I, _P, _I, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P, _I, _I, _I, _P, _I, _P, _P],
     "jllm_moe_gemm_bf16": [_P, _I, _I, _P, _P, _I, _P, _I, _I, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _P],
 }
 
@@ -1193,18 +1197,24 @@ def qkv_prepare(qkv: torch.Tensor, positions: torch.Tensor, slots: Optional[torc
                 gq: Optional[torch.Tensor] = None, gk: Optional[torch.Tensor] = None, eps: float = 0.0,
                 cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, rot_dims: int = 0,
                 temp_coef: float = 0.0, temp_every: int = 0, norm_per_head: bool = False,
-                pairing: str = "interleaved") -> None:
+                pairing: str = "interleaved", head_mul: Optional[torch.Tensor] = None, tied_values: bool = False) -> None:
     """In place on the first columns of ``qkv`` rows [q: heads x maps x dk | k: kv_heads x maps x dk | v: kv_heads x
     dv]: with ``gq``/``gk`` an RMS norm with those gains over the whole of q and the whole of k (``norm_per_head``: over
     every head alone, with gains [dk] shared by the heads); with ``rot_dims`` the rotation of the pairs (2i, 2i + 1)
     (``pairing`` "half": (i, i + rot_dims / 2)) among the first ``rot_dims`` entries of every q and k head by the table
-    rows of the positions; with ``temp_every`` q times 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1); then k and v go to
-    the rows' ``slots`` in the pages (``slots`` None or negative entries: nothing is stored)."""
-    _dev(qkv, positions, slots, gq, gk, cos, sin, k_cache, v_cache)
+    rows of the positions; with ``temp_every`` q times 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1); with ``head_mul``
+    (fp32 [heads]) head h's q times its h-th number; then k and v go to the rows' ``slots`` in the pages (``slots`` None or
+    negative entries: nothing is stored). ``tied_values``: the rows have no v columns, what is stored as values are the k
+    columns as they came (one map per head, dv = dk)."""
+    _dev(qkv, positions, slots, gq, gk, cos, sin, k_cache, v_cache, head_mul)
     _rows2d(qkv, "qkv")
     T = qkv.shape[0]
     q_slots, k_slots = heads * maps, kv_heads * maps
-    if qkv.shape[1] < (q_slots + k_slots) * dk + kv_heads * dv:
+    if head_mul is not None and (head_mul.dtype != torch.float32 or not head_mul.is_contiguous() or head_mul.numel() != heads):
+        raise KernelError(f"the heads' factors must be a contiguous fp32 tensor of {heads} entries")
+    if tied_values and (dv != dk or maps != 1):
+        raise KernelError(f"values that are the keys: key size {dk}, value size {dv}, {maps} maps per head")
+    if qkv.shape[1] < (q_slots + k_slots) * dk + (0 if tied_values else kv_heads * dv):
         raise KernelError(f"qkv rows have {qkv.shape[1]} entries, fewer than q, k and v take")
     _i32(positions, T, "positions")
     _i32(slots, T, "slots")
@@ -1222,14 +1232,14 @@ def qkv_prepare(qkv: torch.Tensor, positions: torch.Tensor, slots: Optional[torc
     _call("jllm_qkv_prepare", _ptr(qkv), qkv.stride(0), _code(qkv.dtype), T, _ptr(positions), _ptr(slots), q_slots, k_slots,
           kv_heads, dk, dv, _ptr(gq), _ptr(gk), gd, float(eps), _ptr(cos), _ptr(sin), int(rot_dims), float(temp_coef),
           int(temp_every), _ptr(k_cache), _ptr(v_cache), k_cache.shape[2], 1 if norm_per_head else 0,
-          1 if pairing == "half" else 0, _stream())
+          1 if pairing == "half" else 0, _ptr(head_mul), int(maps), 1 if tied_values else 0, _stream())
 
 
 def attention_dv(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                  row_req: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, maps: int, dk: int, dv: int,
                  scale: float, *, softcap: float = 0.0, window: int = 0, out_dtype: Optional[torch.dtype] = None,
                  meta=None, exact: bool = False, defer_merge: bool = False, keep_first: int = 0,
-                 sinks: Optional[torch.Tensor] = None):
+                 sinks: Optional[torch.Tensor] = None, chunk: int = 0, slopes: Optional[torch.Tensor] = None):
     """Causal attention of every row of ``q`` [T, heads x maps x dk] over its request's pages, keys [pages, kv_heads x
     maps, page_size, dk] and values [pages, kv_heads, page_size, dv]: map m of head h reads key slot (h / (heads /
     kv_heads)) * maps + m and value head h / (heads / kv_heads). Scores (q . k) * scale, capped as softcap * tanh(score
@@ -1237,8 +1247,14 @@ def attention_dv(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
     ``defer_merge`` a step whose rows were computed in key ranges comes back as a ``SplitHeads`` (the ranges' sums,
     unmerged), which ``heads_finish`` takes in place of the tensor and merges in its prologue. With ``window`` > 0 the
     query at p sees keys p + 1 - window .. p and, with ``keep_first``, the keys before ``keep_first`` as well.
-    ``sinks`` (fp32 [heads], one map per head): exp(sink_h) joins head h's softmax denominator and has no value."""
-    _dev(q, k_cache, v_cache, block_table, row_req, positions, sinks)
+    ``sinks`` (fp32 [heads], one map per head): exp(sink_h) joins head h's softmax denominator and has no value. With
+    ``chunk`` > 0 (in place of a window) the query at p sees the keys at p // chunk * chunk .. p. ``slopes`` (fp32
+    [heads]): slope_h times the distance between query and key is taken off head h's (capped) scores."""
+    _dev(q, k_cache, v_cache, block_table, row_req, positions, sinks, slopes)
+    if slopes is not None and (slopes.dtype != torch.float32 or not slopes.is_contiguous() or slopes.numel() != heads):
+        raise KernelError(f"attention: the slopes must be a contiguous fp32 tensor of {heads} entries")
+    if chunk < 0 or (chunk and window):
+        raise KernelError(f"attention: chunks of {chunk} positions beside a window of {window}")
     if sinks is not None and (sinks.dtype != torch.float32 or not sinks.is_contiguous() or sinks.numel() != heads or maps != 1):
         raise KernelError(f"attention: the sinks must be a contiguous fp32 tensor of {heads} entries (and one map per head)")
     if keep_first < 0:
@@ -1257,7 +1273,7 @@ def attention_dv(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
         return out
     if not exact and _fast_attention_dv is not None:
         got = _fast_attention_dv(q, out, k_cache, v_cache, block_table, row_req, positions, heads, kv_heads, maps, dk, dv, scale,
-                                 softcap, window, meta, defer_merge, keep_first, sinks)
+                                 softcap, window, meta, defer_merge, keep_first, sinks, chunk, slopes)
         if got is not False:
             return out if got is True else got
     if not exact:
@@ -1265,7 +1281,7 @@ def attention_dv(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
     _call("jllm_attention_dv_generic", _ptr(q), q.stride(0), _code(q.dtype), _ptr(out), out.stride(0), _code(out.dtype),
           _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(row_req), _ptr(positions), T, heads,
           kv_heads, maps, dk, dv, k_cache.shape[2], int(window), float(scale), float(softcap), int(keep_first), _ptr(sinks),
-          _stream())
+          int(chunk), _ptr(slopes), _stream())
     return out
 
 
@@ -1281,8 +1297,15 @@ class SplitHeads:
         self.sinks = sinks  # fp32 [heads] or None: joins the denominator when the ranges are merged
 
 
+def visible_blocks(context: int, span: int = 0, keep_first: int = 0) -> int:
+    """The most 64-key blocks that a row may have to read: all of its context's, or, where it sees at most ``span``
+    neighbouring keys (a window or a chunk; they may start anywhere in a block) and the first ``keep_first``, those."""
+    blocks = -(-max(context, 1) // 64)
+    return min(blocks, (span + 62) // 64 + 1 + -(-keep_first // 64)) if span else blocks
+
+
 def _fast_attention_dv(q, out, k_cache, v_cache, block_table, row_req, positions, heads, kv_heads, maps, dk, dv, scale,
-                       softcap, window, meta, defer_merge=False, keep_first=0, sinks=None):
+                       softcap, window, meta, defer_merge=False, keep_first=0, sinks=None, chunk=0, slopes=None):
     """The matrix-core kernel: bf16 pages, fp32 out, and the step's rows cut into tiles by the caller (``meta``:
     "tiles_dev" int32 [n_tiles, 4] as (request, first row, rows, first position or -1), "n_tiles")."""
     tiles = meta.get("tiles_dev") if meta else None
@@ -1294,7 +1317,7 @@ def _fast_attention_dv(q, out, k_cache, v_cache, block_table, row_req, positions
     splits, per_split, partial = 1, 0, None
     T = q.shape[0]
     if meta.get("single_rows") and n_tiles == T:
-        blocks = -(-max(int(meta.get("max_context", 1)), 1) // 64)
+        blocks = visible_blocks(int(meta.get("max_context", 1)), window or chunk, keep_first if window else 0)
         # as many workgroups as are resident at once (two per compute unit; one for the instantiations with keys or
         # values beyond 128, whose LDS buffers fill a unit): a second round would start its chains of loads all over.
         # The heads of a key slot share a workgroup
@@ -1309,7 +1332,7 @@ def _fast_attention_dv(q, out, k_cache, v_cache, block_table, row_req, positions
     ran = _try("jllm_attention_dv_bf16", _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_cache), _ptr(v_cache),
                _ptr(block_table), block_table.shape[1], _ptr(tiles), n_tiles, _ptr(positions), heads, kv_heads, maps, dk, dv,
                k_cache.shape[2], int(window), float(scale), float(softcap), splits, per_split, _ptr(partial),
-               T if meta.get("single_rows") else -1, 1 if defer else 0, int(keep_first), _ptr(sinks), _stream())
+               T if meta.get("single_rows") else -1, 1 if defer else 0, int(keep_first), _ptr(sinks), int(chunk), _ptr(slopes), _stream())
     if ran and defer:
         return SplitHeads(partial, splits, T, heads * maps, dv, sinks)
     return ran
@@ -1514,10 +1537,15 @@ def ssm_scan(xbc: torch.Tensor, proj: torch.Tensor, dt_off: int, a_log: torch.Te
 
 
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float, groups: int,
-                     out_dtype: torch.dtype) -> torch.Tensor:
+                     out_dtype: torch.dtype, *, gate_fn: str = "silu", gate_last: bool = False,
+                     out: Optional[torch.Tensor] = None, out_mul: float = 1.0) -> torch.Tensor:
     """rmsnorm(y * silu(z)) * weight with the root mean square taken over each of ``groups`` equal parts of a row: ``y``
-    fp32 [T, width], ``z`` [T, width] (a view with any row stride), ``weight`` [width]. The gate comes before the norm."""
-    _dev(y, z, weight)
+    fp32 [T, width], ``z`` [T, width] (a view with any row stride), ``weight`` [width]. The gate comes before the norm;
+    ``gate_last``: rmsnorm(y) * weight * gate(z). ``gate_fn``: "silu" or "sigmoid". The result is multiplied by ``out_mul``;
+    ``out``: where to write (a view with any row stride, [T, width]) instead of a new tensor."""
+    if gate_fn not in HEAD_GATES:
+        raise KernelError(f"gated_group_norm: gate function '{gate_fn}' ({sorted(HEAD_GATES)} are built)")
+    _dev(y, z, weight, out)
     _rows2d(y, "rows to norm")
     _rows2d(z, "gate rows")
     T, width = y.shape
@@ -1525,11 +1553,178 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps
         raise KernelError(f"gated_group_norm: fp32 rows {tuple(y.shape)} with a gate of {tuple(z.shape)}")
     if weight.numel() != width or not weight.is_contiguous() or groups <= 0 or width % groups:
         raise KernelError(f"gated_group_norm: a weight of {weight.numel()} for rows of {width} in {groups} groups")
-    out = activation_rows(T, width, out_dtype, y.device)
+    if out is None:
+        out = activation_rows(T, width, out_dtype, y.device)
+    _rows2d(out, "the normed rows")
+    if out.shape != (T, width):
+        raise KernelError(f"gated_group_norm: the output is {tuple(out.shape)}, expected {(T, width)}")
     if T == 0:
         return out
     _call("jllm_gated_group_norm", _ptr(y), y.stride(0), _ptr(z), z.stride(0), _code(z.dtype), _ptr(weight), _code(weight.dtype),
-          float(eps), T, width, int(groups), _ptr(out), _code(out_dtype), out.stride(0), _stream())
+          float(eps), T, width, int(groups), _ptr(out), _code(out.dtype), out.stride(0), HEAD_GATES[gate_fn],
+          1 if gate_last else 0, float(out_mul), _stream())
+    return out
+
+
+# ------------------------------------------------------------------------------------------------ linear attention
+
+MAX_LINEAR_DIM = 256     # state rows per head that the recurrence keeps in registers (csrc/linear_attention.hip)
+LINEAR_CHUNK = 64        # rows of a chunk of the chunked form
+LINEAR_CHUNK_FROM = 24   # a step with a request of at least this many rows takes the chunked form
+
+
+def check_linear_shape(heads: int, dk: int, dv: int, rot_dims: int) -> None:
+    """Raises when the linear-attention kernels do not take these sizes (asked when a model is built)."""
+    if not 0 < heads <= 65535:
+        raise KernelError(f"linear attention: {heads} heads")
+    if not 0 < dk <= MAX_LINEAR_DIM or dv <= 0:
+        raise KernelError(f"linear attention: key size {dk} (1..{MAX_LINEAR_DIM} are taken), value size {dv}")
+    if rot_dims and (rot_dims < 2 or rot_dims > dk or rot_dims % 2):
+        raise KernelError(f"linear attention: a rotary width of {rot_dims} for heads of {dk} (even, 2..{dk}, is taken)")
+
+
+def decay_powers(decay, device) -> torch.Tensor:
+    """d^0 .. d^64 per head from the heads' decays, computed in double: fp32 [heads, 65]."""
+    d = torch.tensor([float(v) for v in decay], dtype=torch.float64)
+    p = torch.ones((d.numel(), LINEAR_CHUNK + 1), dtype=torch.float64)
+    for n in range(1, LINEAR_CHUNK + 1):
+        p[:, n] = torch.pow(d, n)
+    return p.to(torch.float32).to(device).contiguous()
+
+
+def linear_chunk_plan(segments):
+    """The step's rows cut into chunks for ``linear_attention``: (requests int32 [R x 3]: first row, rows, first chunk;
+    chunks int32 [n x 2]: first row, rows) as flat lists, from the step's segments (request order)."""
+    requests, chunks = [], []
+    for s in segments:
+        requests += [s.row0, s.n, len(chunks) // 2]
+        for r in range(0, s.n, LINEAR_CHUNK):
+            chunks += [s.row0 + r, min(LINEAR_CHUNK, s.n - r)]
+    return requests, chunks
+
+
+def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers: torch.Tensor, state: torch.Tensor,
+                     row_req: torch.Tensor, state_slots: torch.Tensor, n_requests: int, heads: int, dk: int, dv: int, *,
+                     positions: Optional[torch.Tensor] = None, cos: Optional[torch.Tensor] = None,
+                     sin: Optional[torch.Tensor] = None, rot_dims: int = 0, silu: bool = False, k_scale: float = 1.0,
+                     requests: Optional[torch.Tensor] = None, chunks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Linear attention with a fixed decay per head over the step's rows, request by request, from and into ``state``
+    [slots, heads, dv, dk] (fp32; a head's matrix S [dk, dv] column by column). ``y`` rows hold q and k (heads x dk) and v
+    (heads x dv) at the given offsets; with ``silu`` all three pass silu; with ``rot_dims`` the pairs (i, i + rot_dims / 2)
+    of every q and k head turn by the table rows of the positions; k is multiplied by ``k_scale``. Per head S <- d S + k
+    v^T, o = S^T q with d from ``powers`` (``decay_powers``). Returns o, fp32 [T, heads x dv]. ``requests`` and ``chunks``
+    (``linear_chunk_plan`` on the device): the chunked form on the matrix cores (fp32), where the sizes allow it; without
+    them the rows are walked one by one."""
+    _dev(y, powers, state, row_req, state_slots, positions, cos, sin, requests, chunks)
+    _rows2d(y, "projection rows")
+    T = y.shape[0]
+    if min(q_off, k_off, v_off) < 0 or max(q_off + heads * dk, k_off + heads * dk, v_off + heads * dv) > y.shape[1]:
+        raise KernelError("linear attention: q, k or v lie outside the projection rows")
+    if powers.dtype != torch.float32 or not powers.is_contiguous() or powers.shape != (heads, LINEAR_CHUNK + 1):
+        raise KernelError(f"linear attention: the decays' powers must be a contiguous fp32 [{heads}, {LINEAR_CHUNK + 1}] tensor")
+    if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 4 or state.shape[1:] != (heads, dv, dk):
+        raise KernelError(f"the state must be a contiguous fp32 [slots, {heads}, {dv}, {dk}] tensor")
+    _i32(row_req, T, "row -> request map")
+    _i32(state_slots, n_requests, "state slots")
+    if rot_dims:
+        if positions is None:
+            raise KernelError("linear attention: a rotation without positions")
+        _i32(positions, T, "positions")
+        _tables(cos, sin, rot_dims)
+    out = torch.empty((T, heads * dv), dtype=torch.float32, device=y.device)
+    if T == 0:
+        return out
+    head = (_ptr(y), y.stride(0), int(q_off), int(k_off), int(v_off), _code(y.dtype), _ptr(positions) if rot_dims else None,
+            _ptr(cos) if rot_dims else None, _ptr(sin) if rot_dims else None, int(rot_dims), 1 if silu else 0, float(k_scale),
+            _ptr(powers), _ptr(state), _ptr(out), out.stride(0))
+    if requests is not None and chunks is not None and requests.numel() and chunks.numel():
+        _i32(requests, 3 * n_requests, "requests of the chunk plan")
+        _i32(chunks, 2, "chunks")
+        n_chunks = chunks.numel() // 2
+        before = torch.empty((n_chunks * heads * dv * dk,), dtype=torch.float32, device=y.device)
+        if _try("jllm_linear_chunks", *head, _ptr(requests), _ptr(chunks), n_chunks, _ptr(before), _ptr(state_slots), T,
+                int(n_requests), heads, dk, dv, _stream()):
+            return out
+    _call("jllm_linear_scan", *head, _ptr(row_req), _ptr(state_slots), T, int(n_requests), heads, dk, dv, _stream())
+    return out
+
+
+# ------------------------------------------------------------------------------------------------ norms on outputs, token shift
+
+
+def _vec32(t: torch.Tensor, n: int, what: str) -> None:
+    if t.dtype != torch.float32 or not t.is_contiguous() or t.numel() != n:
+        raise KernelError(f"{what} must be a contiguous fp32 tensor of {n} entries")
+
+
+def _residual2d(x: torch.Tensor) -> None:
+    if x.dtype != torch.float32 or x.dim() != 2 or not x.is_contiguous():
+        raise KernelError("the residual must be a contiguous fp32 [rows, width] tensor")
+
+
+def _shift_state(state: torch.Tensor, d: int) -> None:
+    if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 2 or state.shape[1] != d:
+        raise KernelError(f"the shift's state must be a contiguous fp32 [slots, {d}] tensor")
+
+
+def rms_seam(residual: torch.Tensor, a: torch.Tensor, gain: torch.Tensor, eps: float, *, a2: Optional[torch.Tensor] = None,
+             branch_gains=None, scales=(1.0, 1.0), branch_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None,
+             shift: Optional[torch.Tensor] = None, state: Optional[torch.Tensor] = None,
+             state_slots: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """``residual += rms(t) * gain`` in one launch, with t = ``a``, or, for two branches, t = scales[0] rms(a) g1 +
+    scales[1] rms(a2) g2 with ``branch_gains`` (g1, g2) and ``branch_eps``. With ``out_dtype`` the new rows come back in that
+    type for the next reader; with ``shift`` (fp32 [width]) as x + (x' - x) shift, x' the request's row in ``state`` [slots,
+    width], which becomes x: for steps in which every request brings one row."""
+    _dev(residual, a, a2, gain, shift, state, state_slots)
+    _residual2d(residual)
+    n, d = residual.shape
+    _vec32(gain, d, "the norm's gain")
+    for t in (a, a2):
+        if t is not None:
+            _rows2d(t, "a sublayer's output")
+            if t.shape != (n, d):
+                raise KernelError(f"rms_seam: a sublayer's output is {tuple(t.shape)}, the residual {(n, d)}")
+    if (a2 is None) != (branch_gains is None):
+        raise KernelError("rms_seam: two branches come with a gain each")
+    if a2 is not None:
+        if a2.dtype != a.dtype:
+            raise KernelError("rms_seam: both branches must share a type")
+        for g in branch_gains:
+            _dev(g)
+            _vec32(g, d, "a branch's gain")
+    if shift is not None:
+        _vec32(shift, d, "the shift")
+        if state is None or state_slots is None or out_dtype is None:
+            raise KernelError("rms_seam: a shift comes with a state, the requests' slots and an output")
+        _shift_state(state, d)
+        _i32(state_slots, n, "state slots")
+    out = activation_rows(n, d, out_dtype, residual.device) if out_dtype is not None else None
+    if n == 0:
+        return out
+    g1, g2 = branch_gains if branch_gains is not None else (None, None)
+    _call("jllm_rms_seam", _ptr(residual), n, d, _ptr(a), a.stride(0), _ptr(a2), a2.stride(0) if a2 is not None else 0, _code(a.dtype),
+          float(scales[0]), float(scales[1]), _ptr(g1), _ptr(g2), float(branch_eps), _ptr(gain), float(eps), _ptr(out),
+          out.stride(0) if out is not None else 0, _code(out.dtype) if out is not None else F32, _ptr(shift), _ptr(state),
+          _ptr(state_slots), _stream())
+    return out
+
+
+def token_shift(h: torch.Tensor, shift: torch.Tensor, state: torch.Tensor, row_req: torch.Tensor, state_slots: torch.Tensor,
+                n_requests: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """h_t + (h_(t-1) - h_t) * shift per row of the step, in ``out_dtype``: h fp32 [T, width], the row before a request's
+    first row of the step is its row of ``state`` [slots, width] (fp32), which then becomes the request's last row."""
+    _dev(h, shift, state, row_req, state_slots)
+    _residual2d(h)
+    T, d = h.shape
+    _vec32(shift, d, "the shift")
+    _shift_state(state, d)
+    _i32(row_req, T, "row -> request map")
+    _i32(state_slots, n_requests, "state slots")
+    out = activation_rows(T, d, out_dtype, h.device)
+    if T == 0:
+        return out
+    _call("jllm_token_shift", _ptr(h), T, int(n_requests), d, _ptr(shift), _ptr(state), _ptr(row_req), _ptr(state_slots), _ptr(out),
+          out.stride(0), _code(out_dtype), _stream())
     return out
 
 

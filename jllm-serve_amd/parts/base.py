@@ -82,6 +82,38 @@ class Part:
         return []
 
 
+class SlotView:
+    """A layer run's slot as one of its parts sees it: the run's pages, and of its state only the part's own tensors."""
+
+    def __init__(self, slot, state):
+        self.group, self.rows, self.page_size, self.writes = slot.group, slot.rows, slot.page_size, slot.writes
+        self.state = state
+
+
+class StateShare:
+    """How the state tensors that a run declares are shared out among its parts: each part's own, in order."""
+
+    def __init__(self, parts):
+        self.specs = []
+        self._at = []  # (first tensor, count, whether the part declared a tuple) per part
+        for p in parts:
+            st = p.state_spec()
+            many = isinstance(st, (tuple, list))
+            own = list(st) if many else [] if st is None else [st]
+            self._at.append((len(self.specs), len(own), many))
+            self.specs += own
+
+    def spec(self):
+        return tuple(self.specs) if self.specs else None
+
+    def view(self, slot, i: int) -> SlotView:
+        at, n, many = self._at[i]
+        if n == 0:
+            return SlotView(slot, None)
+        states = slot.state if isinstance(slot.state, (tuple, list)) else (slot.state,)
+        return SlotView(slot, tuple(states[at:at + n]) if many else states[at])
+
+
 def pad_rows(w: torch.Tensor, multiple: int = 16) -> torch.Tensor:
     """A stacked weight [N, K] (or bias [N]) with zero rows appended up to a multiple of ``multiple``: the product
     kernels for few rows take outputs in whole groups of 16, and a stack that ends in a few per-head rows (two numbers

@@ -16,7 +16,8 @@ import torch
 
 from ..kernels import ops
 from ..weights.loader import WeightSpec
-from .base import Part, part_factory, register_part
+from .base import Part, StateShare, part_factory, register_part
+from .shift import TokenShift
 
 
 class PreNormBlock(Part):
@@ -163,6 +164,7 @@ class SandwichBlock(Part):
         then, vec = (next_norm, add_after) if self.ffn is None else (self.norm_post, None)
         scales = getattr(getattr(self.mixer, "spec", None), "scales", ())
         if hasattr(self.mixer, "outputs") and not getattr(self.mixer, "fused", False) and len(scales) == 2 \
+                and not getattr(self.mixer, "out_names", None) \
                 and hasattr(self.norm_mixer_out, "seam") \
                 and (then is None or hasattr(then, "seam")):
             # two weighted branches: their sum is taken inside the seam's launch
@@ -327,3 +329,100 @@ class HyperBlock(Part):
 
 
 register_part("arrangement", "hyper", HyperBlock, replace=True)
+
+
+class StreamRows:
+    """How the first sublayer of a postnorm layer gets its input from the stream: the rows themselves in the run's type,
+    shifted by a token where the layer has a ``TokenShift``. ``then(step)`` is what the launch that writes the stream is
+    asked for (``norm.join``), or None when it cannot make these rows (``forward`` then does)."""
+
+    def __init__(self, shift, state, dtype):
+        self.shift, self.state, self.dtype = shift, state, dtype
+
+    def then(self, step):
+        if self.shift is None:
+            return {"out_dtype": self.dtype}
+        if not self.shift.rides(step):
+            return None
+        return {"out_dtype": self.dtype, "shift": self.shift.shift, "state": self.state, "state_slots": step.state_slots}
+
+    def forward(self, x, step):
+        return x.to(self.dtype) if self.shift is None else self.shift.forward(x, step, self.state)
+
+
+class PostNormBlock(Part):
+    """A norm behind each sublayer and none in front: x += norm_mixer_out(mixer(x)); x += norm_ffn_out(ffn(x)). The
+    sublayers read the stream itself (rounded to the run's type), the mixer with a token shift where the layer names one.
+    The norm of a sublayer's output (with the branches of a parallel mixer normed and averaged in front of it), its add
+    into the stream and the rows for the next reader are one launch (``norm.join``)."""
+
+    chains_norms = True
+
+    def __init__(self, spec, prefix, build, positions):
+        ending = getattr(spec, "name_ending", ".weight")
+        make = part_factory("norm", spec.norm.kind)
+
+        def norm(name):
+            if not name:
+                raise ValueError(f"{prefix}: the postnorm arrangement names the norm behind each sublayer")
+            part = make(spec.norm, build.hidden, f"{prefix}.{name}{ending}", build)
+            if not hasattr(part, "join"):
+                raise ValueError(f"{prefix}: the postnorm arrangement ends a sublayer in the norm's launch; norm '{spec.norm.kind}' does not offer that")
+            return part
+
+        self.width = build.hidden
+        self.dtype = build.dtype
+        self.shift = TokenShift(f"{prefix}.{spec.token_shift}{ending}", build) if spec.token_shift else None
+        mixer_prefix = f"{prefix}.{spec.mixer_prefix}" if getattr(spec, "mixer_prefix", "") else prefix
+        self.mixer = part_factory("mixer", spec.mixer.kind)(spec.mixer, mixer_prefix, build, positions)
+        self.norm_mixer_out = norm(spec.norm_mixer_out_name)
+        self.ffn = self.norm_ffn_out = None
+        if spec.ffn is not None:
+            self.ffn = part_factory("ffn", spec.ffn.kind)(spec.ffn, prefix, build)
+            self.norm_ffn_out = norm(spec.norm_ffn_out_name)
+        self.parts = tuple(p for p in (self.shift, self.mixer, self.norm_mixer_out, self.ffn, self.norm_ffn_out) if p is not None)
+        self.states = StateShare([p for p in (self.shift, self.mixer) if p is not None])
+        self.capturable = all(getattr(p, "capturable", True) for p in self.parts)
+
+    def weight_specs(self):
+        return [w for p in self.parts for w in p.weight_specs()]
+
+    def load(self, get):
+        for p in self.parts:
+            p.load(get)
+
+    def cache_spec(self):
+        return self.mixer.cache_spec()
+
+    def state_spec(self):
+        return self.states.spec()
+
+    def step_planners(self):
+        return [pl for p in self.parts for pl in (p.step_planners() if hasattr(p, "step_planners") else [])]
+
+    def stream_reader(self, slot):
+        """What reads the stream first in a run of this layer with the state in ``slot``."""
+        return StreamRows(self.shift, self.states.view(slot, 0).state if self.shift is not None else None, self.dtype)
+
+    def _mixed(self, xb, step, slot):
+        """The mixer's output for ``norm.join``: its rows, and how its branches are normed and weighed in front."""
+        view = self.states.view(slot, 1 if self.shift is not None else 0)
+        m = self.mixer
+        gains = getattr(m, "out_gains", None)
+        if gains is not None and len(gains) == 2:
+            return m.outputs(xb, step, view), {"scales": m.spec.scales, "branch_gains": gains, "branch_eps": m.spec.out_eps}
+        return [sublayer_output(m, xb, step, view, self.width)], {}
+
+    def forward(self, x, step, slot, normed_in=None, next_norm=None):
+        """``normed_in``: the mixer's input as the block before left it (a tensor) or None; ``next_norm``: the
+        ``StreamRows`` of the run that follows. Returns its rows of the new x when the last launch made them."""
+        xb = normed_in if isinstance(normed_in, torch.Tensor) else self.stream_reader(slot).forward(x, step)
+        after = next_norm.then(step) if isinstance(next_norm, StreamRows) else None
+        branches, how = self._mixed(xb, step, slot)
+        if self.ffn is None:
+            return self.norm_mixer_out.join(x, branches, then=after, **how)
+        xb = self.norm_mixer_out.join(x, branches, then={"out_dtype": self.dtype}, **how)
+        return self.norm_ffn_out.join(x, [sublayer_output(self.ffn, xb, step, None, self.width)], then=after)
+
+
+register_part("arrangement", "postnorm", PostNormBlock, replace=True)

@@ -156,7 +156,9 @@ class DecoderModel:
             else:
                 nxt_e = schedule[run + 1] if run + 1 < len(schedule) else None
                 nxt = self.layers[nxt_e.layer] if nxt_e is not None else None
-                next_norm = getattr(nxt, "norm_in", None) if getattr(nxt, "chains_norms", False) else None
+                next_norm = None
+                if getattr(nxt, "chains_norms", False):  # a reader may need the state of the run it reads for
+                    next_norm = nxt.stream_reader(slots[run + 1]) if hasattr(nxt, "stream_reader") else getattr(nxt, "norm_in", None)
                 if nxt_e is not None and nxt_e.add_before is not None and nxt_e.mix_before is None and self.watch is None \
                         and getattr(layer, "takes_stream_vector", False):
                     carry = layer.forward(x, step, slots[run], normed_in=carry, next_norm=next_norm,

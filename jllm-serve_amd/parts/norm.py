@@ -1,5 +1,5 @@
-"""RMSNorm: y = (x * rsqrt(mean(x^2) + eps)) * g over fp32 rows (cpu/VectorKernels.java:630-634), layer norm with a
-weight and a bias: y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b, and Dynamic Tanh, which takes no statistics
+"""RMSNorm: y = (x * rsqrt(mean(x^2) + eps)) * g over fp32 rows (cpu/VectorKernels.java:630-634; the gain may be stored
+around zero, g = 1 + w), layer norm with a weight and a bias: y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b, and Dynamic Tanh, which takes no statistics
 of the row: y = tanh(alpha x) w + b."""
 from __future__ import annotations
 
@@ -17,13 +17,16 @@ class RMSNorm(Part):
         self.dim = dim
         self.weight_name = weight_name
         self.out_dtype = build.dtype
+        self.one_plus = bool(getattr(spec, "one_plus", False))
         self.gain = None
 
     def weight_specs(self):
-        return [WeightSpec(self.weight_name, (self.dim,), init="gain")]
+        return [WeightSpec(self.weight_name, (self.dim,), init="bias" if self.one_plus else "gain")]
 
     def load(self, get):
         self.gain = get(self.weight_name)
+        if self.one_plus:  # the stored weight lies around zero; in fp32, since 1 + w has more digits than a bf16 holds
+            self.gain = (self.gain.float() + 1.0).contiguous()
 
     def forward(self, x, rows=None):
         return ops.rmsnorm(x, self.gain, self.eps, self.out_dtype, rows)
@@ -41,6 +44,15 @@ class RMSNorm(Part):
         """residual += a @ w.T (+ bias), and this norm of the result as a promise: the product that makes the new
         residual rows can prepare their norm on its way out (``ops.gemm_add_then_norm``)."""
         return ops.gemm_add_then_norm(a, w, residual, self.gain, self.eps, self.out_dtype, bias=bias, exact=exact)
+
+    def join(self, residual, branches, scales=(1.0, 1.0), branch_gains=None, branch_eps=0.0, then=None):
+        """``residual += this norm of a sublayer's output`` in one launch. ``branches``: the output, or two branches'
+        outputs, each RMS-normed with its gain (``branch_gains``, ``branch_eps``), weighed and added first. ``then``: what
+        the next reader wants of the new rows: keyword arguments of ``ops.rms_seam`` (its type, a token shift), or None."""
+        if self.gain.dtype != torch.float32:
+            self.gain = self.gain.float().contiguous()
+        return ops.rms_seam(residual, branches[0], self.gain, self.eps, a2=branches[1] if len(branches) == 2 else None,
+                            branch_gains=branch_gains, scales=scales, branch_eps=branch_eps, **(then or {}))
 
 
 register_part("norm", "rmsnorm", RMSNorm, replace=True)

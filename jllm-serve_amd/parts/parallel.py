@@ -7,23 +7,20 @@ Branches that say what their input and output products are (``input_projection``
 ``output_weight``, ``heads_width``) share them: one product with the branches' input weights stacked, each branch
 working from its columns of the result and writing its heads, already multiplied by its weight in the sum, into its
 columns of one buffer, and one output product with the branches' output weights side by side, whose result is the
-weighted sum. A decode layer then has two product launches for the mixer instead of four."""
+weighted sum. A decode layer then has two product launches for the mixer instead of four.
+
+With a norm on every branch's output (``spec.out_norms``) the input product is shared and each branch keeps its output
+product; an arrangement that can takes the branches' outputs (``outputs``), norms, weighs and adds them in the launch
+that ends the sublayer."""
 from __future__ import annotations
 
 import torch
 
 from ..config.schema import ParallelMixerSpec
 from ..kernels import ops
-from .base import BuildContext, Part, pad_rows, part_factory, register_part
+from ..weights.loader import WeightSpec
+from .base import BuildContext, Part, StateShare, pad_rows, part_factory, register_part
 from .block import sublayer_output
-
-
-class _BranchSlot:
-    """A layer run's slot as one branch sees it: the run's pages, and of its state only the branch's own tensors."""
-
-    def __init__(self, slot, state):
-        self.group, self.rows, self.page_size, self.writes = slot.group, slot.rows, slot.page_size, slot.writes
-        self.state = state
 
 
 class ParallelMixer(Part):
@@ -41,21 +38,20 @@ class ParallelMixer(Part):
         self.fused = all(hasattr(b, n) for b in self.branches for n in ("input_projection", "heads_rows_from", "output_weight", "heads_width"))
         self.w_in = self.b_in = self.w_o = None
         self._cols = []
-        # which of the run's state tensors belong to which branch
-        self._state_at = []
-        at = 0
-        for b in self.branches:
-            st = b.state_spec()
-            n = 0 if st is None else (len(st) if isinstance(st, (tuple, list)) else 1)
-            self._state_at.append((at, n, isinstance(st, (tuple, list))))
-            at += n
+        self.states = StateShare(self.branches)
+        if spec.out_norms and len(spec.out_norms) != len(spec.branches):
+            raise ValueError(f"{prefix}: {len(spec.out_norms)} output norms for {len(spec.branches)} branches")
+        self.out_names = [f"{prefix}.{n}" for n in spec.out_norms]
+        self.out_gains = None  # fp32, one per branch
 
     def weight_specs(self):
-        return [w for b in self.branches for w in b.weight_specs()]
+        return [w for b in self.branches for w in b.weight_specs()] + \
+            [WeightSpec(n, (self.width,), init="gain") for n in self.out_names]
 
     def load(self, get):
         for b in self.branches:
             b.load(get)
+        self.out_gains = [get(n).float().contiguous() for n in self.out_names] or None
         if not self.fused:
             return
         ins = [b.input_projection() for b in self.branches]
@@ -68,13 +64,13 @@ class ParallelMixer(Part):
         if any(bias is not None for _, bias in ins):
             self.b_in = pad_rows(torch.cat([bias.to(torch.float32) if bias is not None else torch.zeros(w.shape[0], dtype=torch.float32, device=w.device)
                                             for w, bias in ins]).contiguous())
-        self.w_o = torch.cat(outs, dim=1).contiguous()
+        self.w_o = torch.cat(outs, dim=1).contiguous() if self.out_gains is None else None
         at = 0
         for w, _ in ins:
             self._cols.append((at, at + w.shape[0]))
             at += w.shape[0]
         for b in self.branches:  # the stacked copies are the ones that run
-            for name in ("w_in", "b_in", "w_o"):
+            for name in ("w_in", "b_in", "w_o") if self.out_gains is None else ("w_in", "b_in"):
                 if hasattr(b, name):
                     setattr(b, name, None)
 
@@ -82,42 +78,38 @@ class ParallelMixer(Part):
         return next((c for c in (b.cache_spec() for b in self.branches) if c is not None), None)
 
     def state_spec(self):
-        out = []
-        for b in self.branches:
-            st = b.state_spec()
-            if st is not None:
-                out += list(st) if isinstance(st, (tuple, list)) else [st]
-        return tuple(out) if out else None
+        return self.states.spec()
 
     def step_planners(self):
         return [pl for b in self.branches for pl in b.step_planners()]
 
-    def _slot(self, slot, i):
-        at, n, many = self._state_at[i]
-        if n == 0:
-            return _BranchSlot(slot, None)
-        states = slot.state if isinstance(slot.state, (tuple, list)) else (slot.state,)
-        return _BranchSlot(slot, tuple(states[at:at + n]) if many else states[at])
-
     def outputs(self, xb, step, slot):
-        """Every branch's output as fp32 rows, in order (an arrangement may weigh and add them itself)."""
-        if self.fused:
+        """Every branch's output as fp32 rows, in order (an arrangement may norm, weigh and add them itself)."""
+        if not self.fused:
+            return [sublayer_output(b, xb, step, self.states.view(slot, i), self.width) for i, b in enumerate(self.branches)]
+        if self.out_gains is None:
             raise RuntimeError("the branches of this mixer share their products: ask for output()")
-        return [sublayer_output(b, xb, step, self._slot(slot, i), self.width) for i, b in enumerate(self.branches)]
+        exact = self.build.exact
+        y = ops.gemm(xb, self.w_in, bias=self.b_in, out_dtype=self.build.dtype, exact=exact)
+        return [ops.gemm(b.heads_rows_from(y[:, lo:hi], step, self.states.view(slot, i)), b.output_weight(),
+                         out_dtype=torch.float32, exact=exact)
+                for i, (b, (lo, hi)) in enumerate(zip(self.branches, self._cols))]
 
     def output(self, xb, step, slot):
-        if self.fused:
+        if self.fused and self.out_gains is None:
             exact = self.build.exact
             y = ops.gemm(xb, self.w_in, bias=self.b_in, out_dtype=self.build.dtype, exact=exact)
             heads = ops.activation_rows(step.n_tokens, self.w_o.shape[1], self.build.dtype, y.device)
             at = 0
             for i, b in enumerate(self.branches):
                 lo, hi = self._cols[i]
-                b.heads_rows_from(y[:, lo:hi], step, self._slot(slot, i), out=heads[:, at:at + b.heads_width],
+                b.heads_rows_from(y[:, lo:hi], step, self.states.view(slot, i), out=heads[:, at:at + b.heads_width],
                                   out_mul=self.spec.scales[i])
                 at += b.heads_width
             return ops.gemm(heads, self.w_o, out_dtype=torch.float32, exact=exact)
         outs = self.outputs(xb, step, slot)
+        if self.out_gains is not None:
+            outs = [ops.rmsnorm(o, g, self.spec.out_eps, torch.float32).contiguous() for o, g in zip(outs, self.out_gains)]
         total = outs[0].mul_(self.spec.scales[0])
         for o, s in zip(outs[1:], self.spec.scales[1:]):
             total.add_(o, alpha=s)

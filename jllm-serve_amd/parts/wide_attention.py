@@ -2,8 +2,9 @@
 put around the softmax (config/schema.py: WideAttentionSpec): two score maps per head whose outputs are subtracted
 (differential attention), a norm with gains over the whole q and k projections or over every head alone, rotation of
 neighbouring pairs or of the two halves of a head's rotated part, capped scores, a query scale that grows with the
-position, a sliding window that may keep the first keys, a learned sink in the softmax's denominator, an output gate per
-channel or per head.
+position, a factor per head on the scores, a distance penalty per head, a sliding window that may keep the first keys or
+chunks of the sequence, values that are the unnormed keys, a learned sink in the softmax's denominator, an output gate
+per channel or per head.
 
 A step is
   1. one product with the stacked weight [W_q | W_k | W_v | W_g] and the stacked bias (zeros for the gate's rows),
@@ -56,6 +57,10 @@ class WideAttention(Part):
             raise ValueError(f"{prefix}: a sink with {spec.maps} score maps per head")
         if spec.keep_first and not spec.window:
             raise ValueError(f"{prefix}: first keys are kept beside a window, and this mixer has none")
+        if spec.chunk and spec.window:
+            raise ValueError(f"{prefix}: chunks of {spec.chunk} positions beside a window of {spec.window}")
+        if spec.tied_values and (spec.vdim != spec.dim or spec.maps != 1):
+            raise ValueError(f"{prefix}: the values are the keys, so their size {spec.vdim} must be {spec.dim} (with one map per head)")
         self.spec = spec
         self.prefix = prefix
         self.build = build
@@ -69,10 +74,14 @@ class WideAttention(Part):
             raise ValueError(f"{prefix}: {e}") from None
         self.q_dim = spec.heads * spec.maps * spec.dim
         self.k_dim = spec.kv_heads * spec.maps * spec.dim
-        self.v_dim = spec.kv_heads * spec.vdim
+        self.v_dim = 0 if spec.tied_values else spec.kv_heads * spec.vdim  # columns of the projection that hold values
         self.o_dim = spec.heads * spec.vdim
         self.gate_dim = spec.heads if spec.gate_per_head else self.o_dim  # rows of W_g: one per head, or one per channel
         self.sinks = None
+        self.temp = None
+        self.slopes = None
+        if spec.distance_bias:
+            self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / spec.heads) for h in range(spec.heads)], dtype=torch.float32).to(build.device)
         self.w_in = self.b_in = self.w_o = self.g_q = self.g_k = None
         self.lam = 0.0
 
@@ -81,11 +90,12 @@ class WideAttention(Part):
 
     def weight_specs(self):
         s, d, nm = self.spec, self.build.hidden, self.spec.names
-        out = [WeightSpec(self._name("q"), (self.q_dim, d)), WeightSpec(self._name("k"), (self.k_dim, d)),
-               WeightSpec(self._name("v"), (self.v_dim, d))]
+        out = [WeightSpec(self._name("q"), (self.q_dim, d)), WeightSpec(self._name("k"), (self.k_dim, d))]
+        if not s.tied_values:
+            out.append(WeightSpec(self._name("v"), (self.v_dim, d)))
         if s.bias:
             out += [WeightSpec(self._name(n, nm.bias_suffix), (w,), init="bias")
-                    for n, w in (("q", self.q_dim), ("k", self.k_dim), ("v", self.v_dim))]
+                    for n, w in (("q", self.q_dim), ("k", self.k_dim), ("v", self.v_dim)) if w]
         if s.qk_norm == "whole":
             out += [WeightSpec(self._name("q", nm.norm_suffix), (self.q_dim,), init="gain"),
                     WeightSpec(self._name("k", nm.norm_suffix), (self.k_dim,), init="gain")]
@@ -94,6 +104,8 @@ class WideAttention(Part):
                     WeightSpec(self._name("k", nm.norm_suffix), (s.dim,), init="gain")]
         if s.sink:
             out.append(WeightSpec(self._name("sink"), (s.heads,), init="bias"))
+        if s.head_temp:
+            out.append(WeightSpec(self._name("temp"), (s.heads,), init="gain"))
         if s.maps == 2:
             out += [WeightSpec(f"{self.prefix}.{n}", (s.dim,), init="bias") for n in nm.lambda_q + nm.lambda_k]
         if s.out_gate:
@@ -103,19 +115,22 @@ class WideAttention(Part):
 
     def load(self, get):
         s, nm = self.spec, self.spec.names
-        stack = [get(self._name(n)) for n in "qkv"]
+        projections = "qk" if s.tied_values else "qkv"
+        stack = [get(self._name(n)) for n in projections]
         if s.out_gate:
             stack.append(get(self._name("gate")))
         dt = stack[0].dtype if all(t.dtype == stack[0].dtype for t in stack) else torch.float32
         self.w_in = pad_rows(torch.cat([t.to(dt) for t in stack], dim=0).contiguous())  # [q | k | v | g] rows
         del stack
         if s.bias:
-            b = [get(self._name(n, nm.bias_suffix)).to(torch.float32) for n in "qkv"]
+            b = [get(self._name(n, nm.bias_suffix)).to(torch.float32) for n in projections]
             if s.out_gate:
                 b.append(torch.zeros(self.gate_dim, dtype=torch.float32, device=b[0].device))
             self.b_in = pad_rows(torch.cat(b).contiguous())
         if s.sink:
             self.sinks = get(self._name("sink")).float().contiguous()
+        if s.head_temp:  # rides on q: (temp q) . k
+            self.temp = get(self._name("temp")).float().contiguous()
         if s.qk_norm in ("whole", "head"):
             self.g_q, self.g_k = get(self._name("q", nm.norm_suffix)), get(self._name("k", nm.norm_suffix))
             if self.g_q.dtype != self.g_k.dtype:
@@ -129,7 +144,7 @@ class WideAttention(Part):
     def cache_spec(self):
         s = self.spec
         return PageSpec((CacheRow("k", (s.kv_heads * s.maps, s.dim), 1), CacheRow("v", (s.kv_heads, s.vdim), 1)), s.window,
-                        s.keep_first if s.window else 0)
+                        s.keep_first if s.window else 0, s.chunk)
 
     def step_planners(self):
         return [WideStepPlanner()]
@@ -171,12 +186,12 @@ class WideAttention(Part):
         ops.qkv_prepare(y, step.positions, g.slots if slot.writes else None, s.heads, s.kv_heads, s.maps, s.dim, s.vdim,
                         k_cache, v_cache, gq=self.g_q, gk=self.g_k, eps=s.eps, cos=cos, sin=sin, rot_dims=rdims,
                         temp_coef=s.q_temp_coef, temp_every=s.q_temp_every, norm_per_head=s.qk_norm == "head",
-                        pairing=self.pairing)
+                        pairing=self.pairing, head_mul=self.temp, tied_values=s.tied_values)
         meta = self._batch_facts(step)
         att = ops.attention_dv(y[:, :self.q_dim], k_cache, v_cache, g.block_table, step.row_req, step.positions, s.heads,
                                s.kv_heads, s.maps, s.dim, s.vdim, s.scale, softcap=s.softcap, window=s.window,
                                out_dtype=torch.float32, meta=meta, exact=exact, defer_merge=True, keep_first=s.keep_first,
-                               sinks=self.sinks)
+                               sinks=self.sinks, chunk=s.chunk, slopes=self.slopes)
         gate_at = self.q_dim + self.k_dim + self.v_dim
         gate = y[:, gate_at:gate_at + self.gate_dim] if s.out_gate else None
         return ops.heads_finish(att, s.heads, s.maps, s.vdim, self.build.dtype, lam=self.lam, normed=s.maps == 2,
