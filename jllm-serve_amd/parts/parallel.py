@@ -83,15 +83,19 @@ class ParallelMixer(Part):
     def step_planners(self):
         return [pl for b in self.branches for pl in b.step_planners()]
 
+    def _slot(self, slot, i):
+        """The run's slot as branch i sees it."""
+        return self.states.view(slot, i)
+
     def outputs(self, xb, step, slot):
         """Every branch's output as fp32 rows, in order (an arrangement may norm, weigh and add them itself)."""
         if not self.fused:
-            return [sublayer_output(b, xb, step, self.states.view(slot, i), self.width) for i, b in enumerate(self.branches)]
+            return [sublayer_output(b, xb, step, self._slot(slot, i), self.width) for i, b in enumerate(self.branches)]
         if self.out_gains is None:
             raise RuntimeError("the branches of this mixer share their products: ask for output()")
         exact = self.build.exact
         y = ops.gemm(xb, self.w_in, bias=self.b_in, out_dtype=self.build.dtype, exact=exact)
-        return [ops.gemm(b.heads_rows_from(y[:, lo:hi], step, self.states.view(slot, i)), b.output_weight(),
+        return [ops.gemm(b.heads_rows_from(y[:, lo:hi], step, self._slot(slot, i)), b.output_weight(),
                          out_dtype=torch.float32, exact=exact)
                 for i, (b, (lo, hi)) in enumerate(zip(self.branches, self._cols))]
 
@@ -103,7 +107,7 @@ class ParallelMixer(Part):
             at = 0
             for i, b in enumerate(self.branches):
                 lo, hi = self._cols[i]
-                b.heads_rows_from(y[:, lo:hi], step, self.states.view(slot, i), out=heads[:, at:at + b.heads_width],
+                b.heads_rows_from(y[:, lo:hi], step, self._slot(slot, i), out=heads[:, at:at + b.heads_width],
                                   out_mul=self.spec.scales[i])
                 at += b.heads_width
             return ops.gemm(heads, self.w_o, out_dtype=torch.float32, exact=exact)

@@ -2,11 +2,12 @@
 
 GA varies what a layer can vary: both mixers, key heads equal to the heads, a part of them and a single one, chunks
 shorter than a page and longer than a 64-key block, a rotation over a part of the head, value sizes on both sides of the
-key size, decays up to nothing lost (one that keeps nothing is for the recurrence alone: the norm of a head that holds a
-single term leaves the sign of q . k, which rounding decides where the two are orthogonal), a layer without a feed-forward; none of its sizes suits the
-matrix-core kernels. GB has sizes in multiples of 16 / 32 (what those kernels take), chunks that end on and off a 64-key
-block and key sizes in all the chunked recurrence's instantiations. GC has only the recurrent mixer (no pages at all) and
-odd sizes. GD has only the side-by-side mixer, one head on each side, and chunks of a single position.
+key size, decays up to 1, a layer without a feed-forward; none of its sizes suits the matrix-core kernels. (A decay of 0
+is for the recurrence alone: behind the norm of a head that holds a single term only the sign of q . k is left, which
+rounding decides where the two are orthogonal.) GB has sizes in multiples of 16 / 32 (what those kernels take), chunks
+that end on and off a 64-key block and key sizes in all the chunked recurrence's instantiations. GC has only the
+recurrent mixer (no pages at all) and odd sizes. GD has only the side-by-side mixer, one head on each side, and chunks of
+a single position.
 """
 import json
 import os

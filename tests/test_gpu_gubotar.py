@@ -311,7 +311,7 @@ def test_chunk_attention_finds_one_key_within_its_chunk_and_not_beyond(dtype, he
         for n in cuts:
             ctx = runner.prepare([StepEntry("far", [0] * n, [])])
             y = ops.gemm(h[at:at + n].to(DEV), w_in, out_dtype=act, exact=dtype == "float32")
-            slot = model.layers[0].mixer.states.view(model.layers[0].states.view(runner.cache.slots[0], 1), 0)
+            slot = model.layers[0].mixer._slot(model.layers[0].states.view(runner.cache.slots[0], 1), 0)
             rows = left.heads_rows_from(y, ctx, slot)
             got.append(ops.gemm(rows, left.output_weight(), out_dtype=torch.float32, exact=dtype == "float32").cpu())
             runner.cache.commit("far", n)
