@@ -25,6 +25,9 @@ model of the same width, heads, latent and experts.
 `--workload compare --design pivipel [--size 2k|4k]` measures a Pivipel model (several residual streams, Dynamic-Tanh
 norms, windowed attention with a sink or with kept first keys, dense and router-chosen expert layers in turn) beside the
 Miforax model of the same width, heads, window and feed-forwards.
+`--workload compare --design gubotar [--size 2k|4k]` measures a Gubotar model (chunked attention beside linear attention
+with a fixed decay, and retention layers, in turn; norms behind the sublayers, a token shift in front of every mixer)
+beside the Kebepel model of the same width, heads and feed-forward.
 `--workload compare [--size 2k|4k]` is another run altogether: a Miforax model (latent attention with a window, dense
 and table-routed expert layers in turn) beside the closest model the engine had before, a Qwen3 dense model with the
 same width, layers, heads, window and feed-forward width, both with random weights: prefill of 2,048 tokens and
@@ -225,6 +228,60 @@ class KebepelWork:
 
     def pairs(self, T: int) -> float:
         return T * (T + 1) / 2.0
+
+    def flops(self, rows: float, pairs: float, selected: float) -> float:
+        return rows * (2.0 * self.per_row + self.row_flops) + self.pair_flops * pairs + 2.0 * self.V * self.d * selected
+
+
+GUBOTAR_CHUNK = 2048  # positions of an attention chunk: as long as the measured prompts, so that both models see every key
+
+
+def gubotar_config(z: dict) -> dict:
+    """From a Kebepel model's sizes: its attention beside linear attention in the place of its delta rule, and retention in
+    the place of its differential attention, as every second layer's mixer from the second on."""
+    decay = lambda n: [1.0 - 2.0 ** (-5 - 4.0 * h / n) for h in range(n)]
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"], "scale": z["dim"] ** -0.5,
+            "mask": {"size": GUBOTAR_CHUNK}}
+    right = {"heads": z["r_heads"], "dim": z["dim"], "vdim": z["vdim"], "decay": decay(z["r_heads"])}
+    ret = {"heads": z["d_heads"], "dim": z["dim"], "vdim": z["d_vdim"], "decay": decay(z["d_heads"]), "rot": {"base": 1e4, "dims": z["dim"]}}
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    return {"architecture": "Gubotar", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "max_positions": 8192,
+            "layers": [{"type": "retention", "mixer": ret, "mlp": mlp} if i % 2 else
+                       {"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp} for i in range(z["layers"])]}
+
+
+class GubotarWork:
+    """Bytes and flops of passes over a Gubotar model of the sizes ``z`` (the interface of ``Work``). A decode step reads
+    every weight, per request the keys and values (cached as two tensors) of its chunk, and reads and writes the recurrent
+    matrices (fp32); a row costs 2 flops per weight, per (row, key) pair and head 4 dim, and in a recurrence 4 dim vdim
+    per head (the update of the matrix and the read-out)."""
+
+    def __init__(self, z: dict, dtype: str):
+        self.z = z
+        self.L, self.d, self.H, self.Hkv, self.F, self.V, self.hd = z["layers"], z["width"], z["heads"], z["kv_heads"], z["ff"], z["vocab"], z["dim"]
+        self.esize = 2 if dtype == "bf16" else 4
+        self.dtype = dtype
+        d, dk = self.d, z["dim"]
+        left = (2 * z["heads"] + z["kv_heads"]) * dk * d  # q, k and o: the values are the keys
+
+        def linear(heads, dv):
+            return heads * (2 * dk + 3 * dv) * d  # q, k, v, gate and o
+        self.n_ret = self.L // 2
+        self.n_par = self.L - self.n_ret
+        self.per_row = self.n_par * (left + linear(z["r_heads"], z["vdim"])) + self.n_ret * linear(z["d_heads"], z["d_vdim"]) + self.L * 3 * d * z["ff"]
+        self.kv_bytes_per_token = self.n_par * z["kv_heads"] * 2 * dk * self.esize
+        matrices = dk * (self.n_par * z["r_heads"] * z["vdim"] + self.n_ret * z["d_heads"] * z["d_vdim"])
+        self.state_bytes = matrices * 4 * 2
+        self.pair_flops = self.n_par * 4 * z["heads"] * dk
+        self.row_flops = 4 * matrices
+        self.weight_bytes = (self.per_row + self.V * d) * self.esize
+
+    def decode_bytes(self, tokens_held: float, batch: int = 0) -> float:
+        held = min(tokens_held, GUBOTAR_CHUNK * max(batch, 1))
+        return self.weight_bytes + self.kv_bytes_per_token * held + self.state_bytes * max(batch, 1)
+
+    def pairs(self, T: int) -> float:
+        return sum(i % GUBOTAR_CHUNK + 1 for i in range(T))
 
     def flops(self, rows: float, pairs: float, selected: float) -> float:
         return rows * (2.0 * self.per_row + self.row_flops) + self.pair_flops * pairs + 2.0 * self.V * self.d * selected
@@ -437,6 +494,31 @@ def compare_kebepel(args) -> dict:
     return out
 
 
+def compare_gubotar(args) -> dict:
+    """``--workload compare --design gubotar``: the Gubotar model of ``--size`` and the Kebepel model of the same width,
+    heads, head size and feed-forward, one after the other: prefill of 2,048 tokens in one portion, decoding at batch 8
+    and 64 behind prompts of 1,152 tokens."""
+    z = KEBEPEL_SIZES[args.size]
+    ctx = 4096
+    decodes = [dict(key=f"b{B}", batch=B, prompt_len=1152, steps=args.point_steps, warmup=4) for B in (8, 64)]
+    prefills = [dict(key="main", tokens=2048, portion=2048)]
+    out = {"metric": f"Gubotar beside Kebepel at equal sizes ({args.size})", "unit": "tok/s", "n_gpus": 1, "dtype": "bf16",
+           "data": "synthetic (random weights N(0,0.02), uniform-random token ids)", "higher_is_better": True,
+           "config": {"size": args.size, **z, "context": ctx, "page_size": PAGE}, "models": {}}
+    for name, shape, work in (("gubotar", gubotar_config(z), GubotarWork(z, "bf16")), ("kebepel", kebepel_config(z), KebepelWork(z, "bf16"))):
+        r = steady(args, name, "bf16", 0, ctx, decodes, prefills, shape=shape, work=work)
+        m = {"prefill_2048_tok_s": r["prefill"]["main"]["value"], "prefill_2048_ms": r["prefill"]["main"]["ms"],
+             "prefill_flop_frac": r["prefill"]["main"]["frac"]}
+        for B in (8, 64):
+            s_, held, by = r["decode"][f"b{B}"]
+            m[f"decode_b{B}_tok_s"] = round(B / s_, 1)
+            m[f"decode_b{B}_ms"] = round(s_ * 1e3, 3)
+            m[f"decode_b{B}_hbm_frac"] = round(by / s_ / HBM_PEAK, 4)
+        out["models"][name] = m
+    out["value"] = out["models"]["gubotar"]["decode_b8_tok_s"]
+    return out
+
+
 def compare_workload(args) -> dict:
     """``--workload compare``: the Miforax model of ``--size`` and the Qwen3 dense model of the same sizes, one after
     the other: prefill of 2,048 tokens in one portion, decoding at batch 8 and 64 with every window full."""
@@ -584,9 +666,9 @@ def main() -> int:
                     help="steady: timed decode steps at a fixed batch (the default run); serve: a request set run to the end; "
                          "compare: a Miforax model beside the Qwen3 dense model of the same sizes")
     ap.add_argument("--size", default="2k", choices=sorted(COMPARE_SIZES), help="compare: which sizes")
-    ap.add_argument("--design", default="miforax", choices=["miforax", "kebepel", "ratasun", "pivipel"],
+    ap.add_argument("--design", default="miforax", choices=["miforax", "kebepel", "ratasun", "pivipel", "gubotar"],
                     help="compare: which design stands beside the Qwen3 dense model of the same sizes (ratasun and pivipel: "
-                         "beside the Miforax model of the same sizes)")
+                         "beside the Miforax model of the same sizes; gubotar: beside the Kebepel model)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
@@ -596,7 +678,7 @@ def main() -> int:
         print(json.dumps(serve_workload(args)))
         return 0
     if args.workload == "compare":
-        run = {"kebepel": compare_kebepel, "ratasun": compare_ratasun, "pivipel": compare_pivipel}.get(args.design, compare_workload)
+        run = {"kebepel": compare_kebepel, "ratasun": compare_ratasun, "pivipel": compare_pivipel, "gubotar": compare_gubotar}.get(args.design, compare_workload)
         print(json.dumps(run(args)))
         return 0
 

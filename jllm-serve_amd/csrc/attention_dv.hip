@@ -4,7 +4,7 @@
 // the position, a sliding window that may keep the first keys, a sink in the denominator, a gate per channel or per head.
 // fp32 or bf16 storage, all arithmetic in fp32, any sizes. Three kernels:
 //
-//   qkv_prepare      one workgroup per row of the stacked projection [q | k | v]: optional RMS norm with gains over the
+//   qkv_prepare      one workgroup per row of the stacked projection [q | k | v] (or per four heads of a row): optional RMS norm with gains over the
 //                    whole of q and the whole of k (or over every head alone, with gains shared by the heads); optional
 //                    rotation of the pairs (2i, 2i + 1) (or (i, i + rot_dims / 2)) among the first rot_dims entries of
 //                    every q and k head by the row's position; optional q *= 1 + coef * ln(floor((p + 1) / every) + 1);
@@ -43,18 +43,25 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot_dims, float temp_coef, int temp_every,
     T* __restrict__ kcache, T* __restrict__ vcache, int page_size, int norm_per_head, int pair_halves,
     const float* __restrict__ head_mul, int maps, int v_off) {
-  extern __shared__ float sm[];  // q and k of the row
+  extern __shared__ float sm[];  // q and k of the row (of this workgroup's heads)
   __shared__ float red[PREP_THREADS / 64];
   const int t = blockIdx.x;
-  const int nq = q_slots * dk, nk = k_slots * dk, nv = v_heads * dv;
+  const int nv = v_heads * dv;
+  // where nothing spans a whole projection the heads are shared out over gridDim.y workgroups: this one has the slots
+  // s_lo .. s_hi of [q slots | k slots] and its part of the values
+  const int n_slots = q_slots + k_slots;
+  const int s_lo = (int)((long long)n_slots * blockIdx.y / gridDim.y), s_hi = (int)((long long)n_slots * (blockIdx.y + 1) / gridDim.y);
+  const int v_lo = (int)((long long)nv * blockIdx.y / gridDim.y), v_hi = (int)((long long)nv * (blockIdx.y + 1) / gridDim.y);
+  const int nq_here = max(0, min(s_hi, q_slots) - s_lo) * dk, n_here = (s_hi - s_lo) * dk;
   T* row = qkv + (size_t)t * ld;
+  T* mine = row + (size_t)s_lo * dk;
   const int pos = positions[t];
-  for (int i = threadIdx.x; i < nq + nk; i += PREP_THREADS) sm[i] = ldf(row, i);
+  for (int i = threadIdx.x; i < n_here; i += PREP_THREADS) sm[i] = ldf(mine, i);
   __syncthreads();
   if (gq && norm_per_head) {  // every head alone, a wave per head; the gains [dk] are shared by the heads of q (of k)
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    for (int head = wave; head < q_slots + k_slots; head += PREP_THREADS / 64) {
-      float* p = sm + (size_t)head * dk;
+    for (int head = s_lo + wave; head < s_hi; head += PREP_THREADS / 64) {
+      float* p = sm + (size_t)(head - s_lo) * dk;
       float ss = 0.f;
       for (int i = lane; i < dk; i += 64) ss = fmaf(p[i], p[i], ss);
       const float r = norm_scale(wave_sum(ss), dk, eps);
@@ -62,7 +69,8 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
       for (int i = lane; i < dk; i += 64) p[i] = p[i] * r * ldf(g, i);
     }
     __syncthreads();
-  } else if (gq) {  // the norm over a whole projection, before the heads are split
+  } else if (gq) {  // the norm over a whole projection, before the heads are split (one workgroup per row)
+    const int nq = q_slots * dk, nk = k_slots * dk;
     float sq = 0.f, sk = 0.f;
     for (int i = threadIdx.x; i < nq; i += PREP_THREADS) sq = fmaf(sm[i], sm[i], sq);
     for (int i = threadIdx.x; i < nk; i += PREP_THREADS) sk = fmaf(sm[nq + i], sm[nq + i], sk);
@@ -74,7 +82,7 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
   }
   if (rot_dims > 0) {  // a thread owns a pair: nothing else reads or writes it
     const int half = rot_dims >> 1;
-    const int pairs = (q_slots + k_slots) * half;
+    const int pairs = (s_hi - s_lo) * half;
     for (int i = threadIdx.x; i < pairs; i += PREP_THREADS) {
       const int head = i / half, f = i % half;
       float* p = sm + (size_t)head * dk + (pair_halves ? f : 2 * f);
@@ -88,16 +96,16 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
   }
   float temp = 1.0f;
   if (temp_every > 0) temp = 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f);
-  for (int i = threadIdx.x; i < nq; i += PREP_THREADS)
-    stf(row, i, sm[i] * (head_mul ? temp * head_mul[i / (dk * maps)] : temp));
+  for (int i = threadIdx.x; i < nq_here; i += PREP_THREADS)
+    stf(mine, i, sm[i] * (head_mul ? temp * head_mul[(s_lo + i / dk) / maps] : temp));
   const int slot = slots ? slots[t] : -1;
   if (slot < 0) return;  // a row that stores nothing (padding of a step of fixed size; a run that reads another's cache)
   const int page = slot / page_size, off = slot % page_size;
-  for (int i = threadIdx.x; i < nk; i += PREP_THREADS) {
-    const int h = i / dk, e = i % dk;
-    stf(kcache, (((size_t)page * k_slots + h) * page_size + off) * dk + e, sm[nq + i]);
+  for (int i = nq_here + threadIdx.x; i < n_here; i += PREP_THREADS) {
+    const int h = s_lo + i / dk - q_slots, e = i % dk;
+    stf(kcache, (((size_t)page * k_slots + h) * page_size + off) * dk + e, sm[i]);
   }
-  for (int i = threadIdx.x; i < nv; i += PREP_THREADS) {
+  for (int i = v_lo + threadIdx.x; i < v_hi; i += PREP_THREADS) {
     const int h = i / dv, e = i % dv;
     vcache[(((size_t)page * v_heads + h) * page_size + off) * dv + e] = row[v_off + i];
   }
@@ -117,11 +125,15 @@ extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, cons
   if ((gq == nullptr) != (gk == nullptr)) JLLM_FAIL("qkv_prepare: the norm takes gains for both q and k");
   if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims && (!cos_t || !sin_t))) JLLM_FAIL("qkv_prepare: a rotary width of %d for heads of %d", rot_dims, dk);
   if (page_size <= 0) JLLM_FAIL("qkv_prepare: page_size %d", page_size);
-  const size_t smem = (size_t)(q_slots + k_slots) * dk * sizeof(float);
+  // four heads per workgroup (a wave each) where nothing spans a whole projection: a row is then a chain of waits shared
+  // out over several workgroups
+  const int parts = (gq && !norm_per_head) ? 1 : (q_slots + k_slots + PREP_THREADS / 64 - 1) / (PREP_THREADS / 64);
+  if (parts > 65535) JLLM_FAIL("qkv_prepare: %d heads", q_slots + k_slots);
+  const size_t smem = (size_t)((q_slots + k_slots + parts - 1) / parts) * dk * sizeof(float);
   if (smem > 64 * 1024) JLLM_FAIL("qkv_prepare: q and k of a row take %zu bytes of LDS (64 KB are taken)", smem);
   JLLM_DISPATCH_1(dtype, T, {
     JLLM_DISPATCH_1(gain_dtype, TG, {
-      qkv_prepare_kernel<T, TG><<<n_tokens, PREP_THREADS, smem, stream>>>(
+      qkv_prepare_kernel<T, TG><<<dim3(n_tokens, parts), PREP_THREADS, smem, stream>>>(
           (T*)qkv, ld, positions, slots, q_slots, k_slots, v_heads, dk, dv, (const TG*)gq, (const TG*)gk, eps, cos_t, sin_t,
           rot_dims, temp_coef, temp_every, (T*)kcache, (T*)vcache, page_size, norm_per_head, pair_halves, head_mul, maps,
           tied_values ? q_slots * dk : (q_slots + k_slots) * dk);

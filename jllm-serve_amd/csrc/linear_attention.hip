@@ -7,12 +7,13 @@
 //   linear_scan     token by token, for steps of few rows per request and for sizes that the chunked form does not take:
 //                   a workgroup of four waves owns 16 value columns of one head of one request, 16 lanes per column with
 //                   a sixteenth of the state rows each; the state stays in registers while the rows are walked.
-//   linear_states   the chunked form, for portions of prompts: with the decay fixed, C tokens move the state by
-//                   S' = d^C S + sum_t d^(C - 1 - t) k_t v_t^T, one product of a [dk, C] and a [C, dv] matrix. One
-//                   workgroup per (request, head, 16 value columns) walks the request's chunks of 64 rows in order and
-//                   leaves the state in front of every chunk in a scratch array; the last one is the request's new state.
-//   linear_outputs  the rest is independent per chunk and head: o_t = d^(t + 1) S^T q_t + sum_(s <= t) d^(t - s) (q_t .
-//                   k_s) v_s, three matrix products.
+//   The chunked form, for portions of prompts: with the decay fixed, C tokens move the state by
+//   S' = d^C S + sum_t d^(C - 1 - t) k_t v_t^T, one product of a [dk, C] and a [C, dv] matrix, and what a token reads splits
+//   into what the chunk found and what it wrote itself. A request's rows are cut into chunks of 64:
+//   linear_local    per chunk, head and 64 value columns: the chunk's own sum, into a scratch array
+//   linear_combine  per request, head and entry: walks the chunks in order, leaves the state in front of every chunk in
+//                   the place of the chunk's sum; the last one is the request's new state
+//   linear_outputs  per chunk and head: o_t = d^(t + 1) S^T q_t + sum_(s <= t) d^(t - s) (q_t . k_s) v_s, three products
 //   The products of the chunked form are fp32 matrix-core instructions (v_mfma_f32_16x16x4_f32: fp32 operands, fp32
 //   sums), so the two forms differ by the order of their sums only. The powers of a head's decay come from a table
 //   [heads, 65] that the host computes in double.
@@ -52,10 +53,18 @@ struct LinArgs {
   // the chunked form
   const int* requests;  // [requests, 3]: first row, rows, first chunk
   const int* chunks;    // [chunks, 2]: first row, rows
-  float* before;        // [chunks, heads, dv, dk]: the state in front of every chunk
+  float* before;        // [chunks, heads, dv, dk]: a chunk's own sum, then the state in front of it
 };
 
-__device__ __forceinline__ float lin_act(float z, int silu) { return silu ? z / (1.0f + expf(-z)) : z; }
+// bf16 inputs: the hardware's exp2 and reciprocal (each within a unit or two of the last place in fp32)
+template <typename T>
+__device__ __forceinline__ float lin_act(float z, int silu);
+template <>
+__device__ __forceinline__ float lin_act<float>(float z, int silu) { return silu ? z / (1.0f + expf(-z)) : z; }
+template <>
+__device__ __forceinline__ float lin_act<bf16_t>(float z, int silu) {
+  return silu ? z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)) : z;
+}
 
 // thread = cw * 16 + part: column blockIdx.z * 16 + cw, state rows part * E .. + E. C: rows staged at a time
 template <typename T, int E, int C, bool ROT>
@@ -114,11 +123,11 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
       const int i = w % NP;
       const bool own = t < have && i < dk;
       const T* row = y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + (w < NP ? q_at : k_at);
-      float p = lin_act(ldf(row, own ? i : 0), A.silu);
+      float p = lin_act<T>(ldf(row, own ? i : 0), A.silu);
       if (ROT) {
         const bool turns = own && i < A.rot;
         const int f = turns ? (i < half ? i : i - half) : 0;
-        const float o = lin_act(ldf(row, turns ? (i < half ? i + half : i - half) : 0), A.silu);
+        const float o = lin_act<T>(ldf(row, turns ? (i < half ? i + half : i - half) : 0), A.silu);
         const size_t at = (size_t)(pos0 + r0 + (own ? t : 0)) * half + f;
         const float c = A.cos_t[at], s = A.sin_t[at];
         if (turns) p = i < half ? p * c - o * s : p * c + o * s;
@@ -129,7 +138,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
     if (tid < C * LIN_COLS) {
       const int t = tid / LIN_COLS, cc = tid % LIN_COLS;
       const bool own = t < have && col0 + cc < A.dv;
-      const float p = lin_act(ldf(y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + v_at, own ? cc : 0), A.silu);
+      const float p = lin_act<T>(ldf(y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + v_at, own ? cc : 0), A.silu);
       sm[t * ROWF + 2 * NP + cc] = own ? p : 0.f;
     }
     __syncthreads();
@@ -205,8 +214,8 @@ struct HeadUnit {
     const float cc[4] = {c.x, c.y, c.z, c.w}, ss[4] = {s.x, s.y, s.z, s.w};
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      p[e] = lin_act(a.get(e), silu);
-      q[e] = lin_act(b.get(e), silu);
+      p[e] = lin_act<T>(a.get(e), silu);
+      q[e] = lin_act<T>(b.get(e), silu);
       if (ROT && turns) {
         const float u = p[e], v = q[e];
         p[e] = u * cc[e] - v * ss[e];
@@ -220,134 +229,180 @@ struct HeadUnit {
   }
 };
 
-// grid (request, head, 16 value columns), four waves. Wave w accumulates the state rows of its DT tiles of 16; lane l of
-// a tile holds rows 4 (l / 16) .. + 4 of column l % 16.
+// grid (chunk, head, 64 value columns), four waves. Wave w sums the state rows of its DT tiles of 16 for four tiles of
+// value columns; lane l of a tile holds rows 4 (l / 16) .. + 4 of column l % 16.
 template <typename T, int DT, bool ROT>
-__global__ __launch_bounds__(256) void linear_states_kernel(LinArgs A) {
+__global__ __launch_bounds__(256) void linear_local_kernel(LinArgs A) {
   constexpr int DKP = DT * 64;
-  constexpr int KLD = DKP + 16;   // four neighbouring rows of 16 entries lie in different banks
-  constexpr int NU = DKP / 8 * LIN_ROWS / 256;
+  constexpr int KLD = DKP + 16;  // neighbouring rows of 16 entries lie in different banks
+  constexpr int VLD = 64 + 16;
+  constexpr int UN = DKP / 8;
+  constexpr int NU = UN * LIN_ROWS / 256;
   __shared__ __align__(16) float Ks[LIN_ROWS * KLD];
-  __shared__ __align__(16) float Vs[LIN_ROWS * LIN_COLS];
+  __shared__ __align__(16) float Vs[LIN_ROWS * VLD];
   const int tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
-  const int req = blockIdx.x, h = blockIdx.y, col = blockIdx.z * LIN_COLS + l16;
-  const int lo = A.requests[req * 3], n = A.requests[req * 3 + 1], chunk0 = A.requests[req * 3 + 2];
+  const int c = blockIdx.x, h = blockIdx.y, col0 = blockIdx.z * 64;
+  const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
   const int dk = A.dk, dv = A.dv, units = dk >> 3;
-  if (n <= 0) return;
+  const int vcols = min(64, dv - col0);
   const float* pw = A.powers + (size_t)h * LIN_POWERS;
   const T* y = (const T*)A.y;
   const T* kh = y + A.k_off + (size_t)h * dk;
-  const T* vh = y + A.v_off + (size_t)h * dv + blockIdx.z * LIN_COLS;
+  const T* vh = y + A.v_off + (size_t)h * dv + col0;
   const int pos0 = ROT ? A.positions[lo] : 0;
   const int half = A.rot >> 1;
-  float* S_at = A.state + (((size_t)A.state_slots[req] * A.heads + h) * dv + col) * dk;
-  floatx4 S[DT];
-#pragma unroll
-  for (int j = 0; j < DT; ++j) {
-    const int i = (wave * DT + j) * 16 + 4 * g;
-    S[j] = i < dk ? *(const floatx4*)(S_at + i) : floatx4{0.f, 0.f, 0.f, 0.f};
-  }
   HeadUnit<T, ROT> ku[NU];
-  Raw4<T> vu;
-  auto request = [&](int r0) {  // rows beyond the request's last are read from its last
-    const int last = n - 1;
+  Raw4<T> vu[4];
+  float vw[4];
+  // rows and columns beyond the chunk's are read from its last ones and dropped
 #pragma unroll
-    for (int j = 0; j < NU; ++j) {
-      const int idx = tid + 256 * j;
-      const int t = min(r0 + idx / (DKP / 8), last), u = min(idx % (DKP / 8), units - 1);
-      ku[j].load(kh + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
-                 ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
-    }
-    vu.load(vh + (size_t)(lo + min(r0 + (tid >> 2), last)) * A.ld + (tid & 3) * 4);
-  };
-  request(0);
-  for (int r0 = 0, c = chunk0; r0 < n; r0 += LIN_ROWS, ++c) {
-    const int have = min(LIN_ROWS, n - r0);
-    if (r0) __syncthreads();  // the chunk before has been read
+  for (int j = 0; j < NU; ++j) {
+    const int idx = tid + 256 * j;
+    const int t = min(idx / UN, have - 1), u = min(idx % UN, units - 1);
+    ku[j].load(kh + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
+               ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
+  }
 #pragma unroll
-    for (int j = 0; j < NU; ++j) {
-      const int idx = tid + 256 * j;
-      const int t = idx / (DKP / 8), u = idx % (DKP / 8);
-      float* row = Ks + t * KLD;
-      if (u < units) {
-        ku[j].store(row, t < have, A.silu, A.k_scale);
-      } else {  // the padding behind the key size
-        *(float4*)(row + u * 8) = float4{0.f, 0.f, 0.f, 0.f};
-        *(float4*)(row + u * 8 + 4) = float4{0.f, 0.f, 0.f, 0.f};
-      }
-    }
-    {
-      const int t = tid >> 2;
-      const float w = t < have ? pw[max(have - 1 - t, 0)] : 0.f;
-      float v[4];
+  for (int j = 0; j < 4; ++j) {
+    const int t = (tid >> 4) + 16 * j;
+    vu[j].load(vh + (size_t)(lo + min(t, have - 1)) * A.ld + min((tid & 15) * 4, vcols - 4));
+    vw[j] = pw[max(have - 1 - t, 0)];
+  }
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act(vu.get(e), A.silu) * w : 0.f;
-      *(float4*)(Vs + t * LIN_COLS + (tid & 3) * 4) = float4{v[0], v[1], v[2], v[3]};
+  for (int j = 0; j < NU; ++j) {
+    const int idx = tid + 256 * j;
+    const int t = idx / UN, u = idx % UN;
+    float* row = Ks + t * KLD;
+    if (u < units) {
+      ku[j].store(row, t < have, A.silu, A.k_scale);
+    } else {  // the padding behind the key size
+      *(float4*)(row + u * 8) = float4{0.f, 0.f, 0.f, 0.f};
+      *(float4*)(row + u * 8 + 4) = float4{0.f, 0.f, 0.f, 0.f};
     }
-    __syncthreads();
-    if (r0 + LIN_ROWS < n) request(r0 + LIN_ROWS);  // in flight while this chunk is worked through
-    float* S_c = A.before + (((size_t)c * A.heads + h) * dv + col) * dk;
-    const float dC = pw[have];
+  }
 #pragma unroll
-    for (int j = 0; j < DT; ++j) {
-      const int i = (wave * DT + j) * 16 + 4 * g;
-      if (i < dk) *(floatx4*)(S_c + i) = S[j];
-      S[j] *= dC;
-    }
+  for (int j = 0; j < 4; ++j) {
+    const int t = (tid >> 4) + 16 * j;
+    const bool on = t < have && (tid & 15) * 4 < vcols;
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = on ? lin_act<T>(vu[j].get(e), A.silu) * vw[j] : 0.f;
+    *(float4*)(Vs + t * VLD + (tid & 15) * 4) = float4{v[0], v[1], v[2], v[3]};
+  }
+  __syncthreads();
+  floatx4 S[DT][4];
+#pragma unroll
+  for (int j = 0; j < DT; ++j)
+#pragma unroll
+    for (int n = 0; n < 4; ++n) S[j][n] = floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
-    for (int t0 = 0; t0 < LIN_ROWS; t0 += 4) {
-      const float b = Vs[(t0 + g) * LIN_COLS + l16];
+  for (int t0 = 0; t0 < have; t0 += 4) {
+    float a[DT], b[4];
 #pragma unroll
-      for (int j = 0; j < DT; ++j) S[j] = mfma_f32(Ks[(t0 + g) * KLD + (wave * DT + j) * 16 + l16], b, S[j]);
-    }
+    for (int j = 0; j < DT; ++j) a[j] = Ks[(t0 + g) * KLD + (wave * DT + j) * 16 + l16];
+#pragma unroll
+    for (int n = 0; n < 4; ++n) b[n] = Vs[(t0 + g) * VLD + n * 16 + l16];
+#pragma unroll
+    for (int n = 0; n < 4; ++n)
+      if (n * 16 < vcols) {
+#pragma unroll
+        for (int j = 0; j < DT; ++j) S[j][n] = mfma_f32(a[j], b[n], S[j][n]);
+      }
   }
 #pragma unroll
   for (int j = 0; j < DT; ++j) {
     const int i = (wave * DT + j) * 16 + 4 * g;
-    if (i < dk) *(floatx4*)(S_at + i) = S[j];
+    if (i >= dk) continue;
+#pragma unroll
+    for (int n = 0; n < 4; ++n)
+      if (n * 16 < vcols)
+        *(floatx4*)(A.before + (((size_t)c * A.heads + h) * dv + col0 + n * 16 + l16) * dk + i) = S[j][n];
   }
 }
 
-// grid (chunk, head), eight waves. LDS: Q [64][dk], K [64][dk] (later V [64][dv] in its place), P [64][64].
+// grid (1,024 entries, head, request): a thread carries four entries of the state through the request's chunks
+__global__ __launch_bounds__(256) void linear_combine_kernel(LinArgs A) {
+  constexpr int AHEAD = 8;
+  const int h = blockIdx.y, req = blockIdx.z;
+  const size_t n = (size_t)A.dk * A.dv;
+  const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+  if (i >= n) return;
+  const int rows = A.requests[req * 3 + 1], c0 = A.requests[req * 3 + 2];
+  if (rows <= 0) return;
+  const int chunks = (rows + LIN_ROWS - 1) / LIN_ROWS;
+  const float* pw = A.powers + (size_t)h * LIN_POWERS;
+  const float d_full = pw[LIN_ROWS], d_last = pw[rows - (chunks - 1) * LIN_ROWS];
+  float* st = A.state + ((size_t)A.state_slots[req] * A.heads + h) * n + i;
+  const size_t step = (size_t)A.heads * n;
+  float* buf = A.before + ((size_t)c0 * A.heads + h) * n + i;
+  floatx4 S = *(const floatx4*)st;
+  for (int c = 0; c < chunks; c += AHEAD) {
+    floatx4 kv[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) kv[j] = *(const floatx4*)(buf + (size_t)min(c + j, chunks - 1) * step);
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      if (c + j >= chunks) break;
+      *(floatx4*)(buf + (size_t)(c + j) * step) = S;
+      S = (c + j + 1 < chunks ? d_full : d_last) * S + kv[j];
+    }
+  }
+  *(floatx4*)st = S;
+}
+
+// grid (chunk, head), eight waves. LDS: Q [64][dk], the ten tiles of P on and below the diagonal, K [64][dk] (later V
+// [64][dv] in its place).
+#define LIN_PLD 20                     // floats between the rows of a tile of P
+#define LIN_PTILE (16 * LIN_PLD)
 template <typename T, int DT, bool ROT>
 __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
   constexpr int DKP = DT * 64;
   constexpr int QLD = DKP + 4;
-  constexpr int PLD = LIN_ROWS + 4;
   constexpr int UN = DKP / 8;
   constexpr int NU = UN * LIN_ROWS / 512;
+  constexpr int NV = 8;  // pieces of V per thread, for values of up to 256
   extern __shared__ __align__(16) float lin_smem[];
   float* Qs = lin_smem;
   float* Ps = Qs + LIN_ROWS * QLD;
-  float* Ks = Ps + LIN_ROWS * PLD;
+  float* Ks = Ps + 10 * LIN_PTILE;
   const int tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
   const int c = blockIdx.x, h = blockIdx.y;
   const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
-  const int dk = A.dk, dv = A.dv, units = dk >> 3, vld = dv + 4;
+  const int dk = A.dk, dv = A.dv, units = dk >> 3, vld = dv + 4, v4 = dv >> 2;
   const float* pw = A.powers + (size_t)h * LIN_POWERS;
   const T* y = (const T*)A.y;
   const int pos0 = ROT ? A.positions[lo] : 0;
   const int half = A.rot >> 1;
+  {
+    const T* head[2] = {y + A.q_off + (size_t)h * dk, y + A.k_off + (size_t)h * dk};
+    HeadUnit<T, ROT> hu[2][NU];
 #pragma unroll
-  for (int which = 0; which < 2; ++which) {
-    const T* head = y + (which ? A.k_off : A.q_off) + (size_t)h * dk;
-    HeadUnit<T, ROT> hu[NU];
+    for (int which = 0; which < 2; ++which)
 #pragma unroll
-    for (int j = 0; j < NU; ++j) {
-      const int idx = tid + 512 * j;
-      const int t = min(idx / UN, have - 1), u = min(idx % UN, units - 1);
-      hu[j].load(head + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
-                 ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
-    }
+      for (int j = 0; j < NU; ++j) {
+        const int idx = tid + 512 * j;
+        const int t = min(idx / UN, have - 1), u = min(idx % UN, units - 1);
+        hu[which][j].load(head[which] + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
+                          ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
+      }
 #pragma unroll
-    for (int j = 0; j < NU; ++j) {
-      const int idx = tid + 512 * j;
-      const int t = idx / UN, u = idx % UN;
-      if (u < units) hu[j].store((which ? Ks : Qs) + t * QLD, t < have, A.silu, which ? A.k_scale : 1.0f);
-    }
+    for (int which = 0; which < 2; ++which)
+#pragma unroll
+      for (int j = 0; j < NU; ++j) {
+        const int idx = tid + 512 * j;
+        const int t = idx / UN, u = idx % UN;
+        if (u < units) hu[which][j].store((which ? Ks : Qs) + t * QLD, t < have, A.silu, which ? A.k_scale : 1.0f);
+      }
   }
+  Raw4<T> vr[NV];  // in flight while P is computed
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
+    if (512 * j < LIN_ROWS * v4) {
+      const int idx = tid + 512 * j;
+      vr[j].load(y + (size_t)(lo + min(idx / v4, have - 1)) * A.ld + A.v_off + (size_t)h * dv + idx % v4 * 4);
+    }
   __syncthreads();
   // P[i][j] = d^(i - j) (q_i . k_j) for j <= i: ten tiles of 16 x 16
   for (int tile = wave; tile < 10; tile += 8) {
@@ -355,30 +410,34 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
     const int ct = tile - rt * (rt + 1) / 2;
     const float* qa = Qs + (rt * 16 + l16) * QLD + 4 * g;
     const float* kb = Ks + (ct * 16 + l16) * QLD + 4 * g;
-    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
     for (int k0 = 0; k0 < dk; k0 += 16) {
       const floatx4 a = *(const floatx4*)(qa + k0), b = *(const floatx4*)(kb + k0);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) acc = mfma_f32(a[e], b[e], acc);
+      acc = mfma_f32(a[0], b[0], acc);
+      acc2 = mfma_f32(a[1], b[1], acc2);
+      acc = mfma_f32(a[2], b[2], acc);
+      acc2 = mfma_f32(a[3], b[3], acc2);
     }
+    acc += acc2;
     const int j = ct * 16 + l16;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = rt * 16 + 4 * g + e;
-      Ps[i * PLD + j] = j <= i ? acc[e] * pw[i - j] : 0.f;
+      Ps[tile * LIN_PTILE + (4 * g + e) * LIN_PLD + l16] = j <= i ? acc[e] * pw[max(i - j, 0)] : 0.f;
     }
   }
   __syncthreads();  // K has been read: V takes its place
-  for (int idx = tid; idx < LIN_ROWS * (dv >> 2); idx += 512) {
-    const int t = idx / (dv >> 2), e4 = idx % (dv >> 2) * 4;
-    Raw4<T> r;
-    r.load(y + (size_t)(lo + min(t, have - 1)) * A.ld + A.v_off + (size_t)h * dv + e4);
-    float v[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act(r.get(e), A.silu) : 0.f;
-    *(float4*)(Ks + t * vld + e4) = float4{v[0], v[1], v[2], v[3]};
-  }
+  for (int j = 0; j < NV; ++j)
+    if (512 * j < LIN_ROWS * v4) {
+      const int idx = tid + 512 * j;
+      const int t = idx / v4;
+      float v[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act<T>(vr[j].get(e), A.silu) : 0.f;
+      if (t < LIN_ROWS) *(float4*)(Ks + t * vld + idx % v4 * 4) = float4{v[0], v[1], v[2], v[3]};
+    }
   __syncthreads();
   // a wave takes two row tiles (one early, one late: their causal parts add up to the same) of a tile of value columns
   const int rts[2] = {wave & 1, 3 - (wave & 1)};
@@ -388,22 +447,23 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
 #pragma unroll 4
     for (int k0 = 0; k0 < dk; k0 += 16) {
       const floatx4 b = *(const floatx4*)(S_c + k0);
+      floatx4 a[2];
 #pragma unroll
-      for (int r = 0; r < 2; ++r) {
-        const floatx4 a = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k0);
+      for (int r = 0; r < 2; ++r) a[r] = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k0);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], b[e], acc[r]);
-      }
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int r = 0; r < 2; ++r) acc[r] = mfma_f32(a[r][e], b[e], acc[r]);
     }
 #pragma unroll
     for (int r = 0; r < 2; ++r) {
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc[r][e] *= pw[rts[r] * 16 + 4 * g + e + 1];
-      const float* pa = Ps + (rts[r] * 16 + l16) * PLD + 4 * g;
-      for (int j0 = 0; j0 < (rts[r] + 1) * 16; j0 += 16) {
-        const floatx4 a = *(const floatx4*)(pa + j0);
+      const float* pa = Ps + rts[r] * (rts[r] + 1) / 2 * LIN_PTILE + l16 * LIN_PLD + 4 * g;
+      for (int j = 0; j <= rts[r]; ++j) {
+        const floatx4 a = *(const floatx4*)(pa + j * LIN_PTILE);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], Ks[(j0 + 4 * g + e) * vld + ct * 16 + l16], acc[r]);
+        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], Ks[(j * 16 + 4 * g + e) * vld + ct * 16 + l16], acc[r]);
       }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -417,7 +477,7 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
 template <typename T, int DT, bool ROT>
 static int launch_outputs(dim3 grid, hipStream_t stream, const LinArgs& A) {
   const int qld = DT * 64 + 4, vld = A.dv + 4;
-  const size_t smem = (size_t)LIN_ROWS * (qld + (LIN_ROWS + 4) + (qld > vld ? qld : vld)) * sizeof(float);
+  const size_t smem = ((size_t)LIN_ROWS * (qld + (qld > vld ? qld : vld)) + 10 * LIN_PTILE) * sizeof(float);
   static size_t raised = 64 * 1024;
   if (smem > raised) {
     if (smem > 160 * 1024 ||
@@ -495,17 +555,17 @@ extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, i
   if ((ld & 3) || (q_off & 3) || (k_off & 3) || (v_off & 3) || ((uintptr_t)y % bytes4) || ((uintptr_t)state & 15) || ((uintptr_t)before & 15) ||
       (rot && (((uintptr_t)cos_t & 15) || ((uintptr_t)sin_t & 15))))
     return 1;
-  const dim3 sgrid(n_requests, heads, dv / LIN_COLS), ogrid(n_chunks, heads);
+  if (n_requests > 65535) return 1;
+  const dim3 lgrid(n_chunks, heads, (dv + 63) / 64), cgrid((unsigned)(((size_t)dk * dv / 4 + 255) / 256), heads, n_requests), ogrid(n_chunks, heads);
   int rc = 0;
 #define LIN_CHUNKS(DT)                                                                     \
   do {                                                                                     \
-    if (rot) {                                                                             \
-      linear_states_kernel<T, DT, true><<<sgrid, 256, 0, stream>>>(A);                     \
-      rc = launch_outputs<T, DT, true>(ogrid, stream, A);                                  \
-    } else {                                                                               \
-      linear_states_kernel<T, DT, false><<<sgrid, 256, 0, stream>>>(A);                    \
-      rc = launch_outputs<T, DT, false>(ogrid, stream, A);                                 \
-    }                                                                                      \
+    if (rot)                                                                               \
+      linear_local_kernel<T, DT, true><<<lgrid, 256, 0, stream>>>(A);                      \
+    else                                                                                   \
+      linear_local_kernel<T, DT, false><<<lgrid, 256, 0, stream>>>(A);                     \
+    linear_combine_kernel<<<cgrid, 256, 0, stream>>>(A);                                   \
+    rc = rot ? launch_outputs<T, DT, true>(ogrid, stream, A) : launch_outputs<T, DT, false>(ogrid, stream, A); \
   } while (0)
   JLLM_DISPATCH_1(dtype, T, {
     if (dk <= 64)

@@ -248,6 +248,63 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
   }
 }
 
+// The same for one group per row and widths in multiples of four: four neighbouring entries per thread and load, everything
+// requested in front of the sum and kept in registers.
+template <typename T>
+__device__ __forceinline__ void gn_load4(const T* p, float (&v)[4]);
+template <>
+__device__ __forceinline__ void gn_load4<float>(const float* p, float (&v)[4]) {
+  const float4 t = *(const float4*)p;
+  v[0] = t.x, v[1] = t.y, v[2] = t.z, v[3] = t.w;
+}
+template <>
+__device__ __forceinline__ void gn_load4<bf16_t>(const bf16_t* p, float (&v)[4]) {
+  const uint2 t = *(const uint2*)p;
+  v[0] = __uint_as_float(t.x << 16), v[1] = __uint_as_float(t.x & 0xffff0000u);
+  v[2] = __uint_as_float(t.y << 16), v[3] = __uint_as_float(t.y & 0xffff0000u);
+}
+
+template <typename TZ, typename TW, typename TO, int G>
+__global__ __launch_bounds__(256) void gated_row_norm_kernel(const float* __restrict__ y, int ldy, const TZ* __restrict__ z, int ldz,
+                                                             const TW* __restrict__ w, float eps, int width, TO* __restrict__ out,
+                                                             int ldo, int gate_fn, int gate_last, float out_mul) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  float t[G][4], zz[G][4], ww[G][4];
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + 256 * k) * 4, at = min(i, width - 4);
+    gn_load4<float>(y + (size_t)r * ldy + at, t[k]);
+    gn_load4<TZ>(z + (size_t)r * ldz + at, zz[k]);
+    gn_load4<TW>(w + at, ww[k]);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < G; ++k)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float gate = group_gate(zz[k][e], gate_fn);
+      if (!gate_last) t[k][e] *= gate;
+      if ((threadIdx.x + 256 * k) * 4 < width) ss = fmaf(t[k][e], t[k][e], ss);
+      zz[k][e] = gate_last ? gate : 1.0f;
+    }
+  const float s = norm_scale(block_sum<4>(ss, red), width, eps);
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + 256 * k) * 4;
+    if (i >= width) continue;
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = t[k][e] * s * ww[k][e] * zz[k][e] * out_mul;
+    TO* o = out + (size_t)r * ldo + i;
+    if constexpr (sizeof(TO) == 4)
+      *(float4*)o = float4{v[0], v[1], v[2], v[3]};
+    else
+      *(uint2*)o = uint2{(uint32_t)f32_to_bf16(v[0]).bits | ((uint32_t)f32_to_bf16(v[1]).bits << 16),
+                         (uint32_t)f32_to_bf16(v[2]).bits | ((uint32_t)f32_to_bf16(v[3]).bits << 16)};
+  }
+}
+
 // gate_fn: 0 sigmoid, 1 silu
 extern "C" int jllm_gated_group_norm(const float* y, int ldy, const void* z, int ldz, int z_dtype, const void* w, int w_dtype,
                                      float eps, int n_rows, int width, int groups, void* out, int out_dtype, int ldo,
@@ -256,6 +313,30 @@ extern "C" int jllm_gated_group_norm(const float* y, int ldy, const void* z, int
   if (width <= 0 || groups <= 0 || width % groups || groups > 65535) JLLM_FAIL("gated_group_norm: rows of %d in %d groups", width, groups);
   if (ldy < width || ldz < width || ldo < width) JLLM_FAIL("gated_group_norm: short rows");
   if (gate_fn != 0 && gate_fn != 1) JLLM_FAIL("gated_group_norm: gate function %d (0 sigmoid and 1 silu are built)", gate_fn);
+  auto on4 = [](const void* p, int ld, int code) { return ld % 4 == 0 && (uintptr_t)p % (code == JLLM_F32 ? 16 : 8) == 0; };
+  const bool wide = groups == 1 && width % 4 == 0 && width <= 256 * 32 && on4(y, ldy, JLLM_F32) && on4(z, ldz, z_dtype) &&
+                    on4(w, 4, w_dtype) && on4(out, ldo, out_dtype);
+#define GN_LAUNCH(G) \
+  gated_row_norm_kernel<TZ, TW, TO, G><<<n_rows, 256, 0, stream>>>(y, ldy, (const TZ*)z, ldz, (const TW*)w, eps, width, (TO*)out, ldo, gate_fn, gate_last, out_mul)
+  if (wide) {
+    JLLM_DISPATCH_1(z_dtype, TZ, {
+      JLLM_DISPATCH_1(w_dtype, TW, {
+        JLLM_DISPATCH_1(out_dtype, TO, {
+          if (width <= 1024)
+            GN_LAUNCH(1);
+          else if (width <= 2048)
+            GN_LAUNCH(2);
+          else if (width <= 4096)
+            GN_LAUNCH(4);
+          else
+            GN_LAUNCH(8);
+        })
+      })
+    })
+    JLLM_CHECK_LAUNCH("gated_row_norm");
+    return 0;
+  }
+#undef GN_LAUNCH
   JLLM_DISPATCH_1(z_dtype, TZ, {
     JLLM_DISPATCH_1(w_dtype, TW, {
       JLLM_DISPATCH_1(out_dtype, TO, {
