@@ -125,9 +125,10 @@ extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, cons
   if ((gq == nullptr) != (gk == nullptr)) JLLM_FAIL("qkv_prepare: the norm takes gains for both q and k");
   if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims && (!cos_t || !sin_t))) JLLM_FAIL("qkv_prepare: a rotary width of %d for heads of %d", rot_dims, dk);
   if (page_size <= 0) JLLM_FAIL("qkv_prepare: page_size %d", page_size);
-  // four heads per workgroup (a wave each) where nothing spans a whole projection: a row is then a chain of waits shared
-  // out over several workgroups
-  const int parts = (gq && !norm_per_head) ? 1 : (q_slots + k_slots + PREP_THREADS / 64 - 1) / (PREP_THREADS / 64);
+  // with few rows four heads per workgroup (a wave each) where nothing spans a whole projection: a row is a chain of waits,
+  // which is then shared out over several workgroups
+  int parts = (gq && !norm_per_head) ? 1 : (q_slots + k_slots + PREP_THREADS / 64 - 1) / (PREP_THREADS / 64);
+  if (n_tokens > 512 && (size_t)(q_slots + k_slots) * dk * sizeof(float) <= 64 * 1024) parts = 1;  // the rows fill the GPU by themselves
   if (parts > 65535) JLLM_FAIL("qkv_prepare: %d heads", q_slots + k_slots);
   const size_t smem = (size_t)((q_slots + k_slots + parts - 1) / parts) * dk * sizeof(float);
   if (smem > 64 * 1024) JLLM_FAIL("qkv_prepare: q and k of a row take %zu bytes of LDS (64 KB are taken)", smem);

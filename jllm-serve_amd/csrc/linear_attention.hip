@@ -10,7 +10,7 @@
 //   The chunked form, for portions of prompts: with the decay fixed, C tokens move the state by
 //   S' = d^C S + sum_t d^(C - 1 - t) k_t v_t^T, one product of a [dk, C] and a [C, dv] matrix, and what a token reads splits
 //   into what the chunk found and what it wrote itself. A request's rows are cut into chunks of 64:
-//   linear_local    per chunk, head and 64 value columns: the chunk's own sum, into a scratch array
+//   linear_local    per chunk, head and 128 value columns: the chunk's own sum, into a scratch array
 //   linear_combine  per request, head and entry: walks the chunks in order, leaves the state in front of every chunk in
 //                   the place of the chunk's sum; the last one is the request's new state
 //   linear_outputs  per chunk and head: o_t = d^(t + 1) S^T q_t + sum_(s <= t) d^(t - s) (q_t . k_s) v_s, three products
@@ -229,23 +229,24 @@ struct HeadUnit {
   }
 };
 
-// grid (chunk, head, 64 value columns), four waves. Wave w sums the state rows of its DT tiles of 16 for four tiles of
-// value columns; lane l of a tile holds rows 4 (l / 16) .. + 4 of column l % 16.
+// grid (chunk, head, 128 value columns), eight waves. Wave w sums the state rows of its DT tiles of 16 (w % 4) for four
+// tiles of value columns (w / 4); lane l of a tile holds rows 4 (l / 16) .. + 4 of column l % 16.
+#define LIN_LOCAL_COLS 128
 template <typename T, int DT, bool ROT>
-__global__ __launch_bounds__(256) void linear_local_kernel(LinArgs A) {
+__global__ __launch_bounds__(512) void linear_local_kernel(LinArgs A) {
   constexpr int DKP = DT * 64;
   constexpr int KLD = DKP + 16;  // neighbouring rows of 16 entries lie in different banks
-  constexpr int VLD = 64 + 16;
+  constexpr int VLD = LIN_LOCAL_COLS + 16;
   constexpr int UN = DKP / 8;
-  constexpr int NU = UN * LIN_ROWS / 256;
+  constexpr int NU = UN * LIN_ROWS / 512;
   __shared__ __align__(16) float Ks[LIN_ROWS * KLD];
   __shared__ __align__(16) float Vs[LIN_ROWS * VLD];
   const int tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
-  const int c = blockIdx.x, h = blockIdx.y, col0 = blockIdx.z * 64;
+  const int c = blockIdx.x, h = blockIdx.y, col0 = blockIdx.z * LIN_LOCAL_COLS;
   const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
   const int dk = A.dk, dv = A.dv, units = dk >> 3;
-  const int vcols = min(64, dv - col0);
+  const int vcols = min(LIN_LOCAL_COLS, dv - col0);
   const float* pw = A.powers + (size_t)h * LIN_POWERS;
   const T* y = (const T*)A.y;
   const T* kh = y + A.k_off + (size_t)h * dk;
@@ -258,20 +259,20 @@ __global__ __launch_bounds__(256) void linear_local_kernel(LinArgs A) {
   // rows and columns beyond the chunk's are read from its last ones and dropped
 #pragma unroll
   for (int j = 0; j < NU; ++j) {
-    const int idx = tid + 256 * j;
+    const int idx = tid + 512 * j;
     const int t = min(idx / UN, have - 1), u = min(idx % UN, units - 1);
     ku[j].load(kh + (size_t)(lo + t) * A.ld, u, A.rot, ROT ? A.cos_t + (size_t)(pos0 + t) * half : nullptr,
                ROT ? A.sin_t + (size_t)(pos0 + t) * half : nullptr);
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const int t = (tid >> 4) + 16 * j;
-    vu[j].load(vh + (size_t)(lo + min(t, have - 1)) * A.ld + min((tid & 15) * 4, vcols - 4));
+    const int t = (tid >> 5) + 16 * j;
+    vu[j].load(vh + (size_t)(lo + min(t, have - 1)) * A.ld + min((tid & 31) * 4, vcols - 4));
     vw[j] = pw[max(have - 1 - t, 0)];
   }
 #pragma unroll
   for (int j = 0; j < NU; ++j) {
-    const int idx = tid + 256 * j;
+    const int idx = tid + 512 * j;
     const int t = idx / UN, u = idx % UN;
     float* row = Ks + t * KLD;
     if (u < units) {
@@ -283,14 +284,16 @@ __global__ __launch_bounds__(256) void linear_local_kernel(LinArgs A) {
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const int t = (tid >> 4) + 16 * j;
-    const bool on = t < have && (tid & 15) * 4 < vcols;
+    const int t = (tid >> 5) + 16 * j;
+    const bool on = t < have && (tid & 31) * 4 < vcols;
     float v[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) v[e] = on ? lin_act<T>(vu[j].get(e), A.silu) * vw[j] : 0.f;
-    *(float4*)(Vs + t * VLD + (tid & 15) * 4) = float4{v[0], v[1], v[2], v[3]};
+    *(float4*)(Vs + t * VLD + (tid & 31) * 4) = float4{v[0], v[1], v[2], v[3]};
   }
   __syncthreads();
+  const int dk_tile = (wave & 3) * DT, v_tile = (wave >> 2) * 4;
+  if (dk_tile * 16 >= dk || v_tile * 16 >= vcols) return;  // nothing of this wave's is in the matrix
   floatx4 S[DT][4];
 #pragma unroll
   for (int j = 0; j < DT; ++j)
@@ -300,24 +303,24 @@ __global__ __launch_bounds__(256) void linear_local_kernel(LinArgs A) {
   for (int t0 = 0; t0 < have; t0 += 4) {
     float a[DT], b[4];
 #pragma unroll
-    for (int j = 0; j < DT; ++j) a[j] = Ks[(t0 + g) * KLD + (wave * DT + j) * 16 + l16];
+    for (int j = 0; j < DT; ++j) a[j] = Ks[(t0 + g) * KLD + (dk_tile + j) * 16 + l16];
 #pragma unroll
-    for (int n = 0; n < 4; ++n) b[n] = Vs[(t0 + g) * VLD + n * 16 + l16];
+    for (int n = 0; n < 4; ++n) b[n] = Vs[(t0 + g) * VLD + (v_tile + n) * 16 + l16];
 #pragma unroll
     for (int n = 0; n < 4; ++n)
-      if (n * 16 < vcols) {
+      if ((v_tile + n) * 16 < vcols) {
 #pragma unroll
         for (int j = 0; j < DT; ++j) S[j][n] = mfma_f32(a[j], b[n], S[j][n]);
       }
   }
 #pragma unroll
   for (int j = 0; j < DT; ++j) {
-    const int i = (wave * DT + j) * 16 + 4 * g;
+    const int i = (dk_tile + j) * 16 + 4 * g;
     if (i >= dk) continue;
 #pragma unroll
     for (int n = 0; n < 4; ++n)
-      if (n * 16 < vcols)
-        *(floatx4*)(A.before + (((size_t)c * A.heads + h) * dv + col0 + n * 16 + l16) * dk + i) = S[j][n];
+      if ((v_tile + n) * 16 < vcols)
+        *(floatx4*)(A.before + (((size_t)c * A.heads + h) * dv + col0 + (v_tile + n) * 16 + l16) * dk + i) = S[j][n];
   }
 }
 
@@ -362,6 +365,7 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
   constexpr int UN = DKP / 8;
   constexpr int NU = UN * LIN_ROWS / 512;
   constexpr int NV = 8;  // pieces of V per thread, for values of up to 256
+  constexpr int KS = DKP / 16;
   extern __shared__ __align__(16) float lin_smem[];
   float* Qs = lin_smem;
   float* Ps = Qs + LIN_ROWS * QLD;
@@ -403,6 +407,14 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
       const int idx = tid + 512 * j;
       vr[j].load(y + (size_t)(lo + min(idx / v4, have - 1)) * A.ld + A.v_off + (size_t)h * dv + idx % v4 * 4);
     }
+  // the state's part for this wave's first tile of value columns, in flight too; entries beyond dk are read from the last
+  floatx4 sb[KS];
+  auto load_state = [&](int ct) {
+    const float* S_c = A.before + (((size_t)c * A.heads + h) * dv + ct * 16 + l16) * dk + 4 * g;
+#pragma unroll
+    for (int k = 0; k < KS; ++k) sb[k] = *(const floatx4*)(S_c + min(k * 16, dk - 16));
+  };
+  if ((wave >> 1) * 16 < dv) load_state(wave >> 1);
   __syncthreads();
   // P[i][j] = d^(i - j) (q_i . k_j) for j <= i: ten tiles of 16 x 16
   for (int tile = wave; tile < 10; tile += 8) {
@@ -442,19 +454,19 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
   // a wave takes two row tiles (one early, one late: their causal parts add up to the same) of a tile of value columns
   const int rts[2] = {wave & 1, 3 - (wave & 1)};
   for (int ct = wave >> 1; ct * 16 < dv; ct += 4) {
-    const float* S_c = A.before + (((size_t)c * A.heads + h) * dv + ct * 16 + l16) * dk + 4 * g;
     floatx4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-#pragma unroll 4
-    for (int k0 = 0; k0 < dk; k0 += 16) {
-      const floatx4 b = *(const floatx4*)(S_c + k0);
+#pragma unroll
+    for (int k = 0; k < KS; ++k) {
+      if (k * 16 >= dk) break;
       floatx4 a[2];
 #pragma unroll
-      for (int r = 0; r < 2; ++r) a[r] = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k0);
+      for (int r = 0; r < 2; ++r) a[r] = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k * 16);
 #pragma unroll
       for (int e = 0; e < 4; ++e)
 #pragma unroll
-        for (int r = 0; r < 2; ++r) acc[r] = mfma_f32(a[r][e], b[e], acc[r]);
+        for (int r = 0; r < 2; ++r) acc[r] = mfma_f32(a[r][e], sb[k][e], acc[r]);
     }
+    if ((ct + 4) * 16 < dv) load_state(ct + 4);
 #pragma unroll
     for (int r = 0; r < 2; ++r) {
 #pragma unroll
@@ -556,14 +568,14 @@ extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, i
       (rot && (((uintptr_t)cos_t & 15) || ((uintptr_t)sin_t & 15))))
     return 1;
   if (n_requests > 65535) return 1;
-  const dim3 lgrid(n_chunks, heads, (dv + 63) / 64), cgrid((unsigned)(((size_t)dk * dv / 4 + 255) / 256), heads, n_requests), ogrid(n_chunks, heads);
+  const dim3 lgrid(n_chunks, heads, (dv + LIN_LOCAL_COLS - 1) / LIN_LOCAL_COLS), cgrid((unsigned)(((size_t)dk * dv / 4 + 255) / 256), heads, n_requests), ogrid(n_chunks, heads);
   int rc = 0;
 #define LIN_CHUNKS(DT)                                                                     \
   do {                                                                                     \
     if (rot)                                                                               \
-      linear_local_kernel<T, DT, true><<<lgrid, 256, 0, stream>>>(A);                      \
+      linear_local_kernel<T, DT, true><<<lgrid, 512, 0, stream>>>(A);                      \
     else                                                                                   \
-      linear_local_kernel<T, DT, false><<<lgrid, 256, 0, stream>>>(A);                     \
+      linear_local_kernel<T, DT, false><<<lgrid, 512, 0, stream>>>(A);                     \
     linear_combine_kernel<<<cgrid, 256, 0, stream>>>(A);                                   \
     rc = rot ? launch_outputs<T, DT, true>(ogrid, stream, A) : launch_outputs<T, DT, false>(ogrid, stream, A); \
   } while (0)
