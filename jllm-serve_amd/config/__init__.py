@@ -10,6 +10,7 @@ from . import kebepel as _kebepel  # registers "kebepel"
 from . import ratasun as _ratasun  # registers "ratasun"
 from . import pivipel as _pivipel  # registers "pivipel"
 from . import gubotar as _gubotar  # registers "gubotar"
+from . import dazilix as _dazilix  # registers "dazilix"
 
 __all__ = ["ConfigError", "GatedMlpNames", "GatedMlpSpec", "GqaNames", "GqaSpec", "LatentAttentionNames", "LatentAttentionSpec", "TableMoeNames", "TableMoeSpec", "ModelNames", "LayerSpec", "ModelConfig", "NormSpec", "RopeScaling", "RopeSpec",
            "ScheduleEntry", "default_schedule", "entry_for", "load_config", "parse_config", "register_architecture",

@@ -247,7 +247,8 @@ class WideAttentionSpec:
     of its own chunk up to p. ``tied_values``: there is no value projection, the values are the keys as projected, before
     any norm or rotation (``vdim`` is ``dim``). ``head_temp``: head h's scores are multiplied by the h-th number of the
     tensor ``temp`` [heads]. ``distance_bias``: with s_h = 2^(-8 (h + 1) / heads), s_h times the distance between query
-    and key is taken off head h's scores."""
+    and key is taken off head h's scores. ``unit_sink``: a one joins every softmax's denominator (a sink whose score is 0
+    whatever the query, without a tensor)."""
 
     heads: int
     kv_heads: int
@@ -272,6 +273,7 @@ class WideAttentionSpec:
     tied_values: bool = False
     head_temp: bool = False
     distance_bias: bool = False
+    unit_sink: bool = False
     names: WideAttentionNames = WideAttentionNames()
     kind: str = "wide_attention"
 
@@ -371,17 +373,27 @@ class LinearAttentionNames:
     gate: str = "g"
     norm: str = "norm"
     o: str = "o"
+    # the input of a decay that the token chooses: W_up (W_down h) + bias
+    decay_down: str = "a1"
+    decay_up: str = "a2"
+    decay_bias: str = "a2.b"
 
 
 @dataclass(frozen=True)
 class LinearAttentionSpec:
-    """Linear attention with a fixed decay per head: a recurrent mixer without a softmax or a denominator. q and k of
+    """Linear attention: a recurrent mixer without a softmax or a denominator, whose state decays. q and k of
     heads x ``dim`` and v of heads x ``vdim`` are projections of the input, each through ``activation`` (None or "silu");
     ``position``: index of a rotary table applied to q and k (half pairing, the first rotary_dim entries of every head)
     or None; k is multiplied by ``k_scale``. Per head S <- decay_h S + k v^T with S [dim, vdim] from zero, o = S^T q.
     ``norm`` "head": every head's o is divided by its root mean square (no weight); "whole": the concatenated heads are
-    RMS-normed together with a weight (tensor ``norm`` [heads x vdim]); ``eps`` inside the root. Then times
-    ``gate_fn``(W_g h), "silu" or "sigmoid", and through W_o."""
+    RMS-normed together with a weight (tensor ``norm`` [heads x vdim]); "head_gain": every head's o is RMS-normed with one
+    weight that the heads share (tensor ``norm`` [vdim]); ``eps`` inside the root. Then times ``gate_fn``(W_g h), "silu" or
+    "sigmoid", and through W_o.
+
+    ``decay``: one number per head; or, with ``decay_per`` "channel" (gated linear attention; ``decay`` is then empty), one per
+    head, key channel and token: sigmoid(z)^(1 / ``tau``) with z = W_up (W_down h) + bias laid out heads x dim, through a
+    middle of ``decay_rank`` numbers (-1: the checkpoint's to choose). It acts on the rows of S that belong to the key
+    channels: S <- diag(decay) S + k v^T."""
 
     heads: int
     dim: int
@@ -393,6 +405,9 @@ class LinearAttentionSpec:
     k_scale: float = 1.0
     norm: str = "head"
     gate_fn: str = "silu"
+    decay_per: str = "head"
+    tau: float = 1.0
+    decay_rank: int = -1
     names: LinearAttentionNames = LinearAttentionNames()
     kind: str = "linear_attention"
 
@@ -481,6 +496,7 @@ class RoutedMoeNames:
     down: str = "down"
     router: str = "mlp.router"
     correction: str = "mlp.correction"
+    router_bias: str = "mlp.router.b"
     shared_gate: str = "mlp.shared.sg"
     ending: str = ""
 
@@ -496,7 +512,8 @@ class RoutedMoeSpec:
     score is its largest choice score. ``normalize`` False: the weights are the chosen s times ``scale``, not divided by
     their sum. ``shared`` (a GatedMlpSpec or None): a feed-forward that runs for every token and is added; with
     ``shared_gate`` it is first multiplied by sigmoid(W_sg h), one number per token (tensor ``shared_gate`` [1,
-    hidden])."""
+    hidden]). ``router_bias``: the logits are W_router h + bias (tensor ``router_bias`` [experts]). (The softmax over the chosen
+    logits alone is ``score`` "softmax" with ``normalize``: the sum over all experts cancels.)"""
 
     experts: int
     top: int
@@ -512,6 +529,7 @@ class RoutedMoeSpec:
     normalize: bool = True
     shared: Any = None
     shared_gate: bool = False
+    router_bias: bool = False
     names: RoutedMoeNames = RoutedMoeNames()
     kind: str = "routed_moe"
 
@@ -544,6 +562,9 @@ class LayerSpec:
     # arrangement "sandwich": x += norm_mixer_out(mixer(norm_in(x))); x += norm_ffn_out(ffn(norm_post(x)))
     norm_mixer_out_name: str = ""
     norm_ffn_out_name: str = ""
+    # a factor per channel on each sublayer's result behind its output norm (tensors [hidden]; the sandwich arrangement)
+    mixer_scale_name: str = ""
+    ffn_scale_name: str = ""
     mixer_prefix: str = ""  # under the layer's prefix, for mixers whose tensor names are relative to it
     token_shift: str = ""
     # arrangement "hyper": the stream has ``streams`` copies per row; sublayer q reads u = sum_s in[s] x_s, and all
@@ -577,12 +598,14 @@ class ScheduleEntry:
     whose cache this run reads instead of writing one of its own (None = its own cache); ``add_before``: a vector
     that joins the stream right before this run (a layer that runs several times with one set of weights has a cache
     or state per run, and may be told which pass it is in this way); ``mix_before``: the stream is first mixed with the
-    embedding output (before the vector joins)."""
+    embedding output (before the vector joins); ``add_embedding``: the embedding output is added to the stream (before
+    the vector joins)."""
 
     layer: int
     cache_from: Optional[int] = None
     add_before: Optional[StreamVector] = None
     mix_before: Optional[StreamMix] = None
+    add_embedding: bool = False
 
 
 @dataclass(frozen=True)
@@ -626,6 +649,8 @@ class ModelConfig:
                 raise ConfigError(f"schedule entry {i} names layer {e.layer}, the model has {n}")
             if e.cache_from is not None and not 0 <= e.cache_from < i:
                 raise ConfigError(f"schedule entry {i} reads the cache of entry {e.cache_from}, which does not run before it")
+            if e.add_embedding and e.mix_before is not None:
+                raise ConfigError(f"schedule entry {i} both mixes the stream with the embedding output and adds it")
 
     @property
     def num_layers(self) -> int:

@@ -1,5 +1,6 @@
-// Linear attention with a fixed decay per head: S <- d_h S + k v^T, o = S^T q with S [dk, dv] per head, no softmax and no
-// denominator. fp32 or bf16 projections, everything from there on and the state in fp32. q, k and v are columns of one
+// Linear attention with a decay: S <- D S + k v^T, o = S^T q with S [dk, dv] per head, no softmax and no denominator. D is
+// one fixed number per head, or (channel decay) one number per head, key channel and token that acts on the rows of S:
+// alpha = sigmoid(z)^(1 / tau) with z an fp32 product's rows. fp32 or bf16 projections, everything from there on and the state in fp32. q, k and v are columns of one
 // projection's rows; on their way in they pass, as asked, silu (all three), a rotation of the pairs (i, i + rot / 2) among
 // the first rot entries of every q and k head by the row's position, and a constant on k. A request's rows of a step are
 // consecutive and in order (row_req ascends), their positions too.
@@ -17,6 +18,20 @@
 //   The products of the chunked form are fp32 matrix-core instructions (v_mfma_f32_16x16x4_f32: fp32 operands, fp32
 //   sums), so the two forms differ by the order of their sums only. The powers of a head's decay come from a table
 //   [heads, 65] that the host computes in double.
+//
+// With a channel decay the chunked form is the same three steps; what takes the powers' place are products of the chunk's
+// alphas, which are only ever multiplied and never divided by (a ratio of two running products overflows where a token
+// forgets everything). The 64 rows are four tiles of 16; within a tile, with p_i the product of the alphas of the tile's
+// rows up to i, u_j of the rows behind j, and T of all of them:
+//   linear_channel_local    k_j u_j T_(later tiles) takes the place of d^(C - 1 - j) k_j; the chunk's own product per
+//                           channel goes to a scratch array for linear_combine
+//   linear_channel_outputs  between two tiles P[i][j] = sum_c q_ic p_ic T_c(tiles between) u_jc k_jc is one product.
+//                           Within a tile, pairs are taken apart by the highest bit in which their places i > j differ:
+//                           for bit s they lie in the two halves of a block of 2 s rows, and the alphas between them are the
+//                           product up to i of the block's second half times the product behind j of its first half. So
+//                           four products of [second halves] x [first halves], of each of which its own pairs are kept,
+//                           and the diagonal q_i . k_i. A lane holds a row's entries and its 16 neighbours the other
+//                           rows', so the half-block products come from each other by lane permutations.
 //
 // State of one request: [heads, dv, dk] (a head's matrix column by column).
 #include <math.h>
@@ -54,7 +69,25 @@ struct LinArgs {
   const int* requests;  // [requests, 3]: first row, rows, first chunk
   const int* chunks;    // [chunks, 2]: first row, rows
   float* before;        // [chunks, heads, dv, dk]: a chunk's own sum, then the state in front of it
+  // channel decay (powers are then unused)
+  const float* z;       // [rows, ldz]: heads x dk
+  int ldz;
+  float inv_tau;
+  float* chunk_decay;   // [chunks, heads, dk]: the product of a chunk's alphas
 };
+
+// sigmoid(z)^(1 / tau), through its logarithm (log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|)), which no z overflows)
+template <typename T>
+__device__ __forceinline__ float channel_alpha(float z, float inv_tau);
+template <>
+__device__ __forceinline__ float channel_alpha<float>(float z, float inv_tau) {
+  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+}
+template <>
+__device__ __forceinline__ float channel_alpha<bf16_t>(float z, float inv_tau) {
+  const float z2 = 1.4426950408889634f * z;
+  return __builtin_amdgcn_exp2f((fminf(z2, 0.f) - __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(z2)))) * inv_tau);
+}
 
 // bf16 inputs: the hardware's exp2 and reciprocal (each within a unit or two of the last place in fp32)
 template <typename T>
@@ -67,11 +100,13 @@ __device__ __forceinline__ float lin_act<bf16_t>(float z, int silu) {
 }
 
 // thread = cw * 16 + part: column blockIdx.z * 16 + cw, state rows part * E .. + E. C: rows staged at a time
-template <typename T, int E, int C, bool ROT>
+template <typename T, int E, int C, bool ROT, bool CHAN>
 __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
   constexpr int NP = LIN_PARTS * E;          // the key size, padded with zeros
-  constexpr int ROWF = 2 * NP + LIN_COLS + 4;  // q | k | v of the workgroup's columns | -
+  constexpr int VAT = (CHAN ? 3 : 2) * NP;
+  constexpr int ROWF = VAT + LIN_COLS + 4;  // q | k (| alpha) | v of the workgroup's columns | -
   constexpr int NQK = (C * 2 * NP + 255) / 256;
+  constexpr int NAL = (C * NP + 255) / 256;
   __shared__ __align__(16) float sm[C * ROWF];
   const int tid = threadIdx.x;
   const int part = tid & 15, cw = tid >> 4;
@@ -109,7 +144,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
   const T* y = (const T*)A.y;
   const int half = A.rot >> 1;
   const int pos0 = ROT ? A.positions[lo] : 0;
-  const float d = A.powers[(size_t)h * LIN_POWERS + 1];
+  const float d = CHAN ? 0.f : A.powers[(size_t)h * LIN_POWERS + 1];
   const size_t q_at = (size_t)A.q_off + (size_t)h * dk, k_at = (size_t)A.k_off + (size_t)h * dk;
   const size_t v_at = (size_t)A.v_off + (size_t)h * A.dv + col0;
   for (int r0 = 0; r0 < n; r0 += C) {
@@ -135,20 +170,31 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
       if (w >= NP) p *= A.k_scale;
       sm[t * ROWF + w] = own ? p : 0.f;
     }
+    if (CHAN) {
+#pragma unroll
+      for (int j = 0; j < NAL; ++j) {
+        const int idx = tid + 256 * j;
+        if (C * NP % 256 && idx >= C * NP) break;
+        const int t = idx / NP, i = idx % NP;
+        const bool own = t < have && i < dk;
+        const float z = A.z[(size_t)(lo + r0 + (own ? t : 0)) * A.ldz + (size_t)h * dk + (own ? i : 0)];
+        sm[t * ROWF + 2 * NP + i] = own ? channel_alpha<T>(z, A.inv_tau) : 0.f;
+      }
+    }
     if (tid < C * LIN_COLS) {
       const int t = tid / LIN_COLS, cc = tid % LIN_COLS;
       const bool own = t < have && col0 + cc < A.dv;
       const float p = lin_act<T>(ldf(y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + v_at, own ? cc : 0), A.silu);
-      sm[t * ROWF + 2 * NP + cc] = own ? p : 0.f;
+      sm[t * ROWF + VAT + cc] = own ? p : 0.f;
     }
     __syncthreads();
     for (int t = 0; t < have; ++t) {
       const float* row = sm + t * ROWF;
-      const float v = row[2 * NP + cw];
+      const float v = row[VAT + cw];
       float o = 0.f;
 #pragma unroll
       for (int e = 0; e < E; ++e) {
-        S[e] = fmaf(v, row[NP + i0 + e], d * S[e]);
+        S[e] = fmaf(v, row[NP + i0 + e], (CHAN ? row[2 * NP + i0 + e] : d) * S[e]);
         o = fmaf(S[e], row[i0 + e], o);
       }
       o = row16_sum(o);
@@ -325,6 +371,7 @@ __global__ __launch_bounds__(512) void linear_local_kernel(LinArgs A) {
 }
 
 // grid (1,024 entries, head, request): a thread carries four entries of the state through the request's chunks
+template <bool CHAN>
 __global__ __launch_bounds__(256) void linear_combine_kernel(LinArgs A) {
   constexpr int AHEAD = 8;
   const int h = blockIdx.y, req = blockIdx.z;
@@ -335,20 +382,28 @@ __global__ __launch_bounds__(256) void linear_combine_kernel(LinArgs A) {
   if (rows <= 0) return;
   const int chunks = (rows + LIN_ROWS - 1) / LIN_ROWS;
   const float* pw = A.powers + (size_t)h * LIN_POWERS;
-  const float d_full = pw[LIN_ROWS], d_last = pw[rows - (chunks - 1) * LIN_ROWS];
+  const float d_full = CHAN ? 0.f : pw[LIN_ROWS], d_last = CHAN ? 0.f : pw[rows - (chunks - 1) * LIN_ROWS];
+  const float* cd = CHAN ? A.chunk_decay + ((size_t)c0 * A.heads + h) * A.dk + i % A.dk : nullptr;  // dk is a multiple of 16
+  const size_t cd_step = (size_t)A.heads * A.dk;
   float* st = A.state + ((size_t)A.state_slots[req] * A.heads + h) * n + i;
   const size_t step = (size_t)A.heads * n;
   float* buf = A.before + ((size_t)c0 * A.heads + h) * n + i;
   floatx4 S = *(const floatx4*)st;
   for (int c = 0; c < chunks; c += AHEAD) {
-    floatx4 kv[AHEAD];
+    floatx4 kv[AHEAD], dc[AHEAD];
 #pragma unroll
-    for (int j = 0; j < AHEAD; ++j) kv[j] = *(const floatx4*)(buf + (size_t)min(c + j, chunks - 1) * step);
+    for (int j = 0; j < AHEAD; ++j) {
+      kv[j] = *(const floatx4*)(buf + (size_t)min(c + j, chunks - 1) * step);
+      if (CHAN) dc[j] = *(const floatx4*)(cd + (size_t)min(c + j, chunks - 1) * cd_step);
+    }
 #pragma unroll
     for (int j = 0; j < AHEAD; ++j) {
       if (c + j >= chunks) break;
       *(floatx4*)(buf + (size_t)(c + j) * step) = S;
-      S = (c + j + 1 < chunks ? d_full : d_last) * S + kv[j];
+      if (CHAN)
+        S = dc[j] * S + kv[j];
+      else
+        S = (c + j + 1 < chunks ? d_full : d_last) * S + kv[j];
     }
   }
   *(floatx4*)st = S;
@@ -486,6 +541,337 @@ __global__ __launch_bounds__(512) void linear_outputs_kernel(LinArgs A) {
   }
 }
 
+// ---------------------------------------------------------------------------------------------------------------------
+// the chunked form with a channel decay
+
+// the value of another lane of the row of 16: of the partner block of 1, 2, 4 or 8 lanes (of any of its lanes)
+template <int S>
+__device__ __forceinline__ float partner(float v) {
+  constexpr int CTRL = S == 1 ? 0xB1 : S == 2 ? 0x4E : S == 4 ? 0x141 : 0x140;
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
+}
+
+// Products of the alphas of a tile's 16 rows, of which a lane holds one (its place l16 in the row of lanes): up to and with
+// the lane's own row (p), of the rows behind it (u), of all (t); over blocks of 1, 2, 4, 8, 16 rows as `widen` is called.
+struct TileProducts {
+  float p, u, t;
+  __device__ __forceinline__ void start(float alpha) { p = alpha, u = 1.0f, t = alpha; }
+  template <int S>
+  __device__ __forceinline__ void widen(int l16) {  // from blocks of S rows to blocks of 2 S
+    const float o = partner<S>(t);
+    if (l16 & S)
+      p *= o;
+    else
+      u *= o;
+    t *= o;
+  }
+};
+
+// A wave stages the rows of tile wave % 4 in every other group of 16 channels from wave / 4 on; lane l: row l % 16, channels
+// 4 (l / 16) .. + 4 of the group.
+// grid (chunk, head, 128 value columns), eight waves, as linear_local
+template <typename T, int DT>
+__global__ __launch_bounds__(512) void linear_channel_local_kernel(LinArgs A) {
+  constexpr int DKP = DT * 64;
+  constexpr int KLD = DKP + 16;
+  constexpr int VLD = LIN_LOCAL_COLS + 16;
+  constexpr int NB = DKP / 32;  // groups of 16 channels per wave
+  __shared__ __align__(16) float Ks[LIN_ROWS * KLD];
+  __shared__ __align__(16) float Vs[LIN_ROWS * VLD];
+  __shared__ __align__(16) float Tot[4 * DKP];
+  const int tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
+  const int c = blockIdx.x, h = blockIdx.y, col0 = blockIdx.z * LIN_LOCAL_COLS;
+  const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
+  const int dk = A.dk, dv = A.dv;
+  const int vcols = min(LIN_LOCAL_COLS, dv - col0);
+  const T* y = (const T*)A.y;
+  const T* vh = y + A.v_off + (size_t)h * dv + col0;
+  const int rt = wave & 3, b0 = wave >> 2;
+  const int row = rt * 16 + l16;
+  const bool on = row < have;
+  const size_t at = (size_t)(lo + min(row, have - 1));  // rows beyond the chunk's are read from its last one and dropped
+  Raw4<T> ku[NB], vu[4];
+  float4 zu[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    const int i = min((b0 + 2 * b) * 16, dk - 16) + 4 * g;
+    ku[b].load(y + at * A.ld + A.k_off + (size_t)h * dk + i);
+    zu[b] = *(const float4*)(A.z + at * A.ldz + (size_t)h * dk + i);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int t = (tid >> 5) + 16 * j;
+    vu[j].load(vh + (size_t)(lo + min(t, have - 1)) * A.ld + min((tid & 31) * 4, vcols - 4));
+  }
+  float u[NB][4];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    const float zz[4] = {zu[b].x, zu[b].y, zu[b].z, zu[b].w};
+    float tot[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      TileProducts tp;
+      tp.start(on ? channel_alpha<T>(zz[e], A.inv_tau) : 1.0f);
+      tp.widen<1>(l16);
+      tp.widen<2>(l16);
+      tp.widen<4>(l16);
+      tp.widen<8>(l16);
+      u[b][e] = tp.u;
+      tot[e] = tp.t;
+    }
+    if (l16 == 0) *(float4*)(Tot + rt * DKP + (b0 + 2 * b) * 16 + 4 * g) = float4{tot[0], tot[1], tot[2], tot[3]};
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int t = (tid >> 5) + 16 * j;
+    const bool von = t < have && (tid & 31) * 4 < vcols;
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = von ? lin_act<T>(vu[j].get(e), A.silu) : 0.f;
+    *(float4*)(Vs + t * VLD + (tid & 31) * 4) = float4{v[0], v[1], v[2], v[3]};
+  }
+  __syncthreads();
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    const int i = (b0 + 2 * b) * 16 + 4 * g;
+    floatx4 w = {u[b][0], u[b][1], u[b][2], u[b][3]};
+    for (int r = rt + 1; r < 4; ++r) w *= *(const floatx4*)(Tot + r * DKP + i);
+    float k[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) k[e] = on && i < dk ? lin_act<T>(ku[b].get(e), A.silu) * A.k_scale * w[e] : 0.f;
+    *(float4*)(Ks + row * KLD + i) = float4{k[0], k[1], k[2], k[3]};
+  }
+  if (blockIdx.z == 0 && tid < dk)
+    A.chunk_decay[((size_t)c * A.heads + h) * dk + tid] = (Tot[tid] * Tot[DKP + tid]) * (Tot[2 * DKP + tid] * Tot[3 * DKP + tid]);
+  __syncthreads();
+  const int dk_tile = (wave & 3) * DT, v_tile = (wave >> 2) * 4;
+  if (dk_tile * 16 >= dk || v_tile * 16 >= vcols) return;  // nothing of this wave's is in the matrix
+  floatx4 S[DT][4];
+#pragma unroll
+  for (int j = 0; j < DT; ++j)
+#pragma unroll
+    for (int n = 0; n < 4; ++n) S[j][n] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int t0 = 0; t0 < have; t0 += 4) {
+    float a[DT], b[4];
+#pragma unroll
+    for (int j = 0; j < DT; ++j) a[j] = Ks[(t0 + g) * KLD + (dk_tile + j) * 16 + l16];
+#pragma unroll
+    for (int n = 0; n < 4; ++n) b[n] = Vs[(t0 + g) * VLD + (v_tile + n) * 16 + l16];
+#pragma unroll
+    for (int n = 0; n < 4; ++n)
+      if ((v_tile + n) * 16 < vcols) {
+#pragma unroll
+        for (int j = 0; j < DT; ++j) S[j][n] = mfma_f32(a[j], b[n], S[j][n]);
+      }
+  }
+#pragma unroll
+  for (int j = 0; j < DT; ++j) {
+    const int i = (dk_tile + j) * 16 + 4 * g;
+    if (i >= dk) continue;
+#pragma unroll
+    for (int n = 0; n < 4; ++n)
+      if ((v_tile + n) * 16 < vcols)
+        *(floatx4*)(A.before + (((size_t)c * A.heads + h) * dv + col0 + (v_tile + n) * 16 + l16) * dk + i) = S[j][n];
+  }
+}
+
+// the pairs of level S (i > j, highest differing bit S) of a tile: the product of the second halves' rows, each times the
+// alphas of its half up to it, with the first halves' rows, each times the alphas of its half behind it; accumulated over
+// four channels
+template <int S>
+__device__ __forceinline__ void level_product(const float (&q)[4], const float (&k)[4], TileProducts (&tp)[4], int l16, floatx4& acc) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const bool second = l16 & S;
+    acc = mfma_f32(second ? q[e] * tp[e].p : 0.f, second ? 0.f : k[e] * tp[e].u, acc);
+    tp[e].widen<S>(l16);
+  }
+}
+
+// grid (chunk, head), eight waves. LDS: Q [64][dk], the ten tiles of P on and below the diagonal, the tiles' products
+// [4][dk], K [64][dk] (later V [64][dv] in its place).
+template <typename T, int DT>
+__global__ __launch_bounds__(512) void linear_channel_outputs_kernel(LinArgs A) {
+  constexpr int DKP = DT * 64;
+  constexpr int QLD = DKP + 4;
+  constexpr int NB = DKP / 32;
+  constexpr int NV = 8;  // pieces of V per thread, for values of up to 256
+  constexpr int KS = DKP / 16;
+  extern __shared__ __align__(16) float lin_smem[];
+  float* Qs = lin_smem;
+  float* Ps = Qs + LIN_ROWS * QLD;
+  float* Tot = Ps + 10 * 256;
+  float* Ks = Tot + 4 * DKP;
+  const int tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
+  const int c = blockIdx.x, h = blockIdx.y;
+  const int lo = A.chunks[c * 2], have = A.chunks[c * 2 + 1];
+  const int dk = A.dk, dv = A.dv, vld = dv + 4, v4 = dv >> 2;
+  const T* y = (const T*)A.y;
+  const int rt = wave & 3, b0 = wave >> 2;
+  const int row = rt * 16 + l16;
+  const bool on = row < have;
+  float qh[NB][4];  // this lane's row: q times the alphas of the tile up to the row
+  floatx4 dg;       // the tile's pairs, this wave's channels
+  {
+    const size_t at = (size_t)(lo + min(row, have - 1));
+    Raw4<T> qu[NB], ku[NB];
+    float4 zu[NB];
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int i = min((b0 + 2 * b) * 16, dk - 16) + 4 * g;
+      qu[b].load(y + at * A.ld + A.q_off + (size_t)h * dk + i);
+      ku[b].load(y + at * A.ld + A.k_off + (size_t)h * dk + i);
+      zu[b] = *(const float4*)(A.z + at * A.ldz + (size_t)h * dk + i);
+    }
+    floatx4 acc1 = {0.f, 0.f, 0.f, 0.f}, acc2 = acc1, acc4 = acc1, acc8 = acc1;
+    float own = 0.f;  // q_i . k_i
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int i = (b0 + 2 * b) * 16 + 4 * g;
+      const float zz[4] = {zu[b].x, zu[b].y, zu[b].z, zu[b].w};
+      const bool in = on && i < dk;
+      float q[4], k[4];
+      TileProducts tp[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        q[e] = in ? lin_act<T>(qu[b].get(e), A.silu) : 0.f;
+        k[e] = in ? lin_act<T>(ku[b].get(e), A.silu) * A.k_scale : 0.f;
+        own = fmaf(q[e], k[e], own);
+        tp[e].start(on ? channel_alpha<T>(zz[e], A.inv_tau) : 1.0f);
+      }
+      level_product<1>(q, k, tp, l16, acc1);
+      level_product<2>(q, k, tp, l16, acc2);
+      level_product<4>(q, k, tp, l16, acc4);
+      level_product<8>(q, k, tp, l16, acc8);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) qh[b][e] = q[e] * tp[e].p;
+      if (i < dk) {
+        *(float4*)(Qs + row * QLD + i) = float4{qh[b][0], qh[b][1], qh[b][2], qh[b][3]};
+        *(float4*)(Ks + row * QLD + i) = float4{k[0] * tp[0].u, k[1] * tp[1].u, k[2] * tp[2].u, k[3] * tp[3].u};
+        if (l16 == 0) *(float4*)(Tot + rt * DKP + i) = float4{tp[0].t, tp[1].t, tp[2].t, tp[3].t};
+      }
+    }
+    own += __shfl_xor(own, 16, 64);
+    own += __shfl_xor(own, 32, 64);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {  // place (i, j) = (4 g + e, l16)
+      const int i = 4 * g + e, x = i ^ l16;
+      const float v = x >= 8 ? acc8[e] : x >= 4 ? acc4[e] : x >= 2 ? acc2[e] : x >= 1 ? acc1[e] : own;
+      dg[e] = i >= l16 ? v : 0.f;
+      if (b0 == 0) Ps[(rt * (rt + 3) / 2) * 256 + i * 16 + l16] = dg[e];
+    }
+  }
+  Raw4<T> vr[NV];  // in flight while P is computed
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
+    if (512 * j < LIN_ROWS * v4) {
+      const int idx = tid + 512 * j;
+      vr[j].load(y + (size_t)(lo + min(idx / v4, have - 1)) * A.ld + A.v_off + (size_t)h * dv + idx % v4 * 4);
+    }
+  // the state's part for this wave's first tile of value columns, in flight too; entries beyond dk are read from the last
+  floatx4 sb[KS];
+  auto load_state = [&](int ct) {
+    const float* S_c = A.before + (((size_t)c * A.heads + h) * dv + ct * 16 + l16) * dk + 4 * g;
+#pragma unroll
+    for (int k = 0; k < KS; ++k) sb[k] = *(const floatx4*)(S_c + min(k * 16, dk - 16));
+  };
+  if ((wave >> 1) * 16 < dv) load_state(wave >> 1);
+  __syncthreads();
+  if (b0 == 1) {  // the other half of the channels
+#pragma unroll
+    for (int e = 0; e < 4; ++e) Ps[(rt * (rt + 3) / 2) * 256 + (4 * g + e) * 16 + l16] += dg[e];
+  }
+  // the six tiles below the diagonal: waves 0 .. 5
+  if (wave < 6) {
+    const int r = wave < 1 ? 1 : wave < 3 ? 2 : 3, ct = wave - r * (r - 1) / 2;
+    const float* qa = Qs + (r * 16 + l16) * QLD + 4 * g;
+    const float* kb = Ks + (ct * 16 + l16) * QLD + 4 * g;
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k0 = 0; k0 < dk; k0 += 16) {
+      floatx4 a = *(const floatx4*)(qa + k0);
+      const floatx4 b = *(const floatx4*)(kb + k0);
+      for (int m = ct + 1; m < r; ++m) a *= *(const floatx4*)(Tot + m * DKP + k0 + 4 * g);
+      acc = mfma_f32(a[0], b[0], acc);
+      acc2 = mfma_f32(a[1], b[1], acc2);
+      acc = mfma_f32(a[2], b[2], acc);
+      acc2 = mfma_f32(a[3], b[3], acc2);
+    }
+    acc += acc2;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) Ps[(r * (r + 1) / 2 + ct) * 256 + (4 * g + e) * 16 + l16] = acc[e];
+  }
+  __syncthreads();  // Q and K have been read: V takes K's place, Q gets the alphas of the tiles before
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    const int i = (b0 + 2 * b) * 16 + 4 * g;
+    if (i >= dk) continue;
+    floatx4 w = {qh[b][0], qh[b][1], qh[b][2], qh[b][3]};
+    for (int m = 0; m < rt; ++m) w *= *(const floatx4*)(Tot + m * DKP + i);
+    *(floatx4*)(Qs + row * QLD + i) = w;
+  }
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
+    if (512 * j < LIN_ROWS * v4) {
+      const int idx = tid + 512 * j;
+      const int t = idx / v4;
+      float v[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = t < have ? lin_act<T>(vr[j].get(e), A.silu) : 0.f;
+      if (t < LIN_ROWS) *(float4*)(Ks + t * vld + idx % v4 * 4) = float4{v[0], v[1], v[2], v[3]};
+    }
+  __syncthreads();
+  // a wave takes two row tiles (one early, one late: their causal parts add up to the same) of a tile of value columns
+  const int rts[2] = {wave & 1, 3 - (wave & 1)};
+  for (int ct = wave >> 1; ct * 16 < dv; ct += 4) {
+    floatx4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int k = 0; k < KS; ++k) {
+      if (k * 16 >= dk) break;
+      floatx4 a[2];
+#pragma unroll
+      for (int r = 0; r < 2; ++r) a[r] = *(const floatx4*)(Qs + (rts[r] * 16 + l16) * QLD + 4 * g + k * 16);
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int r = 0; r < 2; ++r) acc[r] = mfma_f32(a[r][e], sb[k][e], acc[r]);
+    }
+    if ((ct + 4) * 16 < dv) load_state(ct + 4);
+#pragma unroll
+    for (int r = 0; r < 2; ++r) {
+      const float* pa = Ps + rts[r] * (rts[r] + 1) / 2 * 256 + l16 * 16 + 4 * g;
+      for (int j = 0; j <= rts[r]; ++j) {
+        const floatx4 a = *(const floatx4*)(pa + j * 256);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[r] = mfma_f32(a[e], Ks[(j * 16 + 4 * g + e) * vld + ct * 16 + l16], acc[r]);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = rts[r] * 16 + 4 * g + e;
+        if (t < have) A.out[(size_t)(lo + t) * A.ldo + (size_t)h * dv + ct * 16 + l16] = acc[r][e];
+      }
+    }
+  }
+}
+
+template <typename T, int DT>
+static int launch_channel_outputs(dim3 grid, hipStream_t stream, const LinArgs& A) {
+  const int qld = DT * 64 + 4, vld = A.dv + 4;
+  const size_t smem = ((size_t)LIN_ROWS * (qld + (qld > vld ? qld : vld)) + 10 * 256 + 4 * DT * 64) * sizeof(float);
+  static size_t raised = 64 * 1024;
+  if (smem > raised) {
+    if (smem > 160 * 1024 ||
+        hipFuncSetAttribute((const void*)linear_channel_outputs_kernel<T, DT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess)
+      return -1;
+    raised = 160 * 1024;
+  }
+  linear_channel_outputs_kernel<T, DT><<<grid, 512, smem, stream>>>(A);
+  return 0;
+}
+
 template <typename T, int DT, bool ROT>
 static int launch_outputs(dim3 grid, hipStream_t stream, const LinArgs& A) {
   const int qld = DT * 64 + 4, vld = A.dv + 4;
@@ -510,30 +896,38 @@ static int check_args(const char* name, const LinArgs& A, int n_requests) {
     JLLM_FAIL("%s: short rows", name);
   if (A.rot < 0 || A.rot % 2 || A.rot > A.dk || (A.rot && (!A.cos_t || !A.sin_t || !A.positions)))
     JLLM_FAIL("%s: a rotary width of %d for heads of %d", name, A.rot, A.dk);
+  if ((A.z == nullptr) == (A.powers == nullptr)) JLLM_FAIL("%s: a decay per head or per channel", name);
+  if (A.z && (A.ldz < A.heads * A.dk || !(A.inv_tau > 0.f) || A.rot))
+    JLLM_FAIL("%s: decay rows of %d for %d heads of %d (1 / tau %g, rotary width %d)", name, A.ldz, A.heads, A.dk, (double)A.inv_tau, A.rot);
   return 0;
 }
 
 extern "C" int jllm_linear_scan(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
                                 const float* cos_t, const float* sin_t, int rot, int silu, float k_scale, const float* powers,
                                 float* state, float* out, int ldo, const int* row_req, const int* state_slots, int n_rows,
-                                int n_requests, int heads, int dk, int dv, hipStream_t stream) {
+                                int n_requests, int heads, int dk, int dv, const float* z, int ldz, float inv_tau,
+                                hipStream_t stream) {
   if (n_rows <= 0) return 0;
   LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, row_req, state_slots,
-            n_rows, heads, dk, dv, nullptr, nullptr, nullptr};
+            n_rows, heads, dk, dv, nullptr, nullptr, nullptr, z, ldz, inv_tau, nullptr};
   if (check_args("linear_scan", A, n_requests) != 0) return -1;
   dim3 grid(n_requests, heads, (dv + LIN_COLS - 1) / LIN_COLS);
   const int per_lane = (dk + LIN_PARTS - 1) / LIN_PARTS;
   const bool few = n_rows <= 2 * n_requests;
 #define LIN_LAUNCH(E)                                                             \
   do {                                                                            \
-    if (few && rot)                                                               \
-      linear_scan_kernel<T, E, 2, true><<<grid, 256, 0, stream>>>(A);             \
+    if (z && few)                                                                 \
+      linear_scan_kernel<T, E, 2, false, true><<<grid, 256, 0, stream>>>(A);      \
+    else if (z)                                                                   \
+      linear_scan_kernel<T, E, 16, false, true><<<grid, 256, 0, stream>>>(A);     \
+    else if (few && rot)                                                          \
+      linear_scan_kernel<T, E, 2, true, false><<<grid, 256, 0, stream>>>(A);      \
     else if (few)                                                                 \
-      linear_scan_kernel<T, E, 2, false><<<grid, 256, 0, stream>>>(A);            \
+      linear_scan_kernel<T, E, 2, false, false><<<grid, 256, 0, stream>>>(A);     \
     else if (rot)                                                                 \
-      linear_scan_kernel<T, E, 16, true><<<grid, 256, 0, stream>>>(A);            \
+      linear_scan_kernel<T, E, 16, true, false><<<grid, 256, 0, stream>>>(A);     \
     else                                                                          \
-      linear_scan_kernel<T, E, 16, false><<<grid, 256, 0, stream>>>(A);           \
+      linear_scan_kernel<T, E, 16, false, false><<<grid, 256, 0, stream>>>(A);    \
   } while (0)
   JLLM_DISPATCH_1(dtype, T, {
     if (per_lane <= 2)
@@ -551,15 +945,17 @@ extern "C" int jllm_linear_scan(const void* y, int ld, int q_off, int k_off, int
 }
 
 // Returns 1 (declined) for sizes that the chunked form does not take. requests [n_requests, 3]: first row, rows, first
-// chunk; chunks [n_chunks, 2]: first row, rows (at most 64, of one request, in order); before: fp32 [n_chunks, heads, dv, dk]
+// chunk; chunks [n_chunks, 2]: first row, rows (at most 64, of one request, in order); before: fp32 [n_chunks, heads, dv, dk];
+// with z (a channel decay, powers null) chunk_decay: fp32 [n_chunks, heads, dk]
 extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
                                   const float* cos_t, const float* sin_t, int rot, int silu, float k_scale,
                                   const float* powers, float* state, float* out, int ldo, const int* requests,
                                   const int* chunks, int n_chunks, float* before, const int* state_slots, int n_rows,
-                                  int n_requests, int heads, int dk, int dv, hipStream_t stream) {
+                                  int n_requests, int heads, int dk, int dv, const float* z, int ldz, float inv_tau,
+                                  float* chunk_decay, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, nullptr, state_slots,
-            n_rows, heads, dk, dv, requests, chunks, before};
+            n_rows, heads, dk, dv, requests, chunks, before, z, ldz, inv_tau, chunk_decay};
   if (check_args("linear_chunks", A, n_requests) != 0) return -1;
   if (n_chunks < n_requests || n_chunks > n_rows || !requests || !chunks || !before) JLLM_FAIL("linear_chunks: %d chunks of %d rows of %d requests", n_chunks, n_rows, n_requests);
   const size_t bytes4 = dtype == JLLM_F32 ? 16 : 8;
@@ -568,15 +964,23 @@ extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, i
       (rot && (((uintptr_t)cos_t & 15) || ((uintptr_t)sin_t & 15))))
     return 1;
   if (n_requests > 65535) return 1;
+  if (z && ((ldz & 3) || ((uintptr_t)z & 15) || ((uintptr_t)chunk_decay & 15))) return 1;
+  if (z && !chunk_decay) JLLM_FAIL("linear_chunks: no place for the chunks' decays");
   const dim3 lgrid(n_chunks, heads, (dv + LIN_LOCAL_COLS - 1) / LIN_LOCAL_COLS), cgrid((unsigned)(((size_t)dk * dv / 4 + 255) / 256), heads, n_requests), ogrid(n_chunks, heads);
   int rc = 0;
 #define LIN_CHUNKS(DT)                                                                     \
   do {                                                                                     \
+    if (z) {                                                                               \
+      linear_channel_local_kernel<T, DT><<<lgrid, 512, 0, stream>>>(A);                    \
+      linear_combine_kernel<true><<<cgrid, 256, 0, stream>>>(A);                           \
+      rc = launch_channel_outputs<T, DT>(ogrid, stream, A);                                \
+      break;                                                                               \
+    }                                                                                      \
     if (rot)                                                                               \
       linear_local_kernel<T, DT, true><<<lgrid, 512, 0, stream>>>(A);                      \
     else                                                                                   \
       linear_local_kernel<T, DT, false><<<lgrid, 512, 0, stream>>>(A);                     \
-    linear_combine_kernel<<<cgrid, 256, 0, stream>>>(A);                                   \
+    linear_combine_kernel<false><<<cgrid, 256, 0, stream>>>(A);                            \
     rc = rot ? launch_outputs<T, DT, true>(ogrid, stream, A) : launch_outputs<T, DT, false>(ogrid, stream, A); \
   } while (0)
   JLLM_DISPATCH_1(dtype, T, {

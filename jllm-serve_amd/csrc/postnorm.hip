@@ -1,6 +1,9 @@
-// What lies between two sublayers when the norm sits on a sublayer's output and the sublayers read the stream itself, and
-// the mix of a row with the previous token's row.
+// What lies between two sublayers when a norm sits on a sublayer's output, and the mix of a row with the previous token's
+// row.
 //
+//   rms_between   for sublayers that are normed on both sides. Per row, each part optional: t = s1 a (+ s2 a2) and x +=
+//                 rms(t) g; x += the row's further row (the embedding output); x += a vector; and the norm of the new row
+//                 for the next sublayer's products, rms(x) g'.
 //   rms_seam      per row: t = a, or, for two branches side by side, t = s1 rms(a) w1 + s2 rms(a2) w2; the residual row
 //                 x += rms(t) g; and the new row for the next reader: as it is, or shifted, x + (x' - x) mu with x' the
 //                 request's previous row. The shifted form is for steps in which every request brings one row: x' is
@@ -153,6 +156,132 @@ __global__ __launch_bounds__(PN_THREADS) void rms_seam_kernel(SeamArgs A) {
 }
 
 static bool pn_aligned(const void* p, size_t bytes) { return ((uintptr_t)p % bytes) == 0; }
+
+struct BetweenArgs {
+  float* x;  // [rows, d]
+  int d;
+  const void* a;  // [rows, lda] or null
+  int lda;
+  const void* a2;  // or null
+  int lda2;
+  float s1, s2;
+  const float* gain;  // with a
+  float eps;
+  const float* rows;  // [rows, d] or null
+  const void* vec;    // [d] or null
+  int vec_bf16;
+  const float* gain_next;  // with out
+  float eps_next;
+  void* out;  // [rows, ldo] or null
+  int ldo;
+};
+
+template <typename TA, typename TO, int V, int G>
+__global__ __launch_bounds__(PN_THREADS) void rms_between_kernel(BetweenArgs A) {
+  __shared__ float red[2 * (PN_THREADS / 64)];
+  const int r = blockIdx.x, d = A.d;
+  float* xr = A.x + (size_t)r * d;
+  const TA* a = A.a ? (const TA*)A.a + (size_t)r * A.lda : nullptr;
+  const TA* a2 = A.a2 ? (const TA*)A.a2 + (size_t)r * A.lda2 : nullptr;
+  // everything the row needs is requested before the first sum
+  float x[G][V], t[G][V], u[G][V], gn[G][V], more[G][V], vec[G][V], nx[G][V];
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PN_THREADS) * V;
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[k][e] = t[k][e] = u[k][e] = gn[k][e] = more[k][e] = vec[k][e] = nx[k][e] = 0.f;
+    if (i >= d) continue;
+    pn_load<V>(xr + i, x[k]);
+    if (a) {
+      pn_load<V>(a + i, t[k]);
+      pn_load<V>(A.gain + i, gn[k]);
+      if (a2) pn_load<V>(a2 + i, u[k]);
+    }
+    if (A.rows) pn_load<V>(A.rows + (size_t)r * d + i, more[k]);
+    if (A.vec) {
+      if (A.vec_bf16)
+        pn_load<V>((const bf16_t*)A.vec + i, vec[k]);
+      else
+        pn_load<V>((const float*)A.vec + i, vec[k]);
+    }
+    if (A.out) pn_load<V>(A.gain_next + i, nx[k]);
+  }
+  if (a) {
+    float q = 0.f;
+#pragma unroll
+    for (int k = 0; k < G; ++k)
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        t[k][e] = a2 ? fmaf(A.s2, u[k][e], A.s1 * t[k][e]) : A.s1 * t[k][e];
+        q = fmaf(t[k][e], t[k][e], q);
+      }
+    const float rs = norm_scale(pn_block_sum(q, red), d, A.eps);
+#pragma unroll
+    for (int k = 0; k < G; ++k)
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[k][e] += t[k][e] * rs * gn[k][e];
+  }
+  float q = 0.f;
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PN_THREADS) * V;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      x[k][e] = (x[k][e] + more[k][e]) + vec[k][e];
+      q = fmaf(x[k][e], x[k][e], q);
+    }
+    if (i < d && (a || A.rows || A.vec)) pn_store<V>(xr + i, x[k]);
+  }
+  if (!A.out) return;
+  const float rs = norm_scale(pn_block_sum(q, red + PN_THREADS / 64), d, A.eps_next);
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PN_THREADS) * V;
+    if (i >= d) continue;
+    float o[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) o[e] = x[k][e] * rs * nx[k][e];
+    pn_store<V>((TO*)A.out + (size_t)r * A.ldo + i, o);
+  }
+}
+
+// a, a2 in a_dtype, the vector in vec_dtype; gains and rows fp32
+extern "C" int jllm_rms_between(float* x, int n, int d, const void* a, int lda, const void* a2, int lda2, int a_dtype, float s1,
+                                float s2, const float* gain, float eps, const float* rows, const void* vec, int vec_dtype,
+                                const float* gain_next, float eps_next, void* out, int ldo, int out_dtype, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (d <= 0 || d > PN_THREADS * 32) JLLM_FAIL("rms_between: rows of %d entries (1..%d are taken)", d, PN_THREADS * 32);
+  if (!x || (a && (!gain || lda < d)) || (a2 && (!a || lda2 < d))) JLLM_FAIL("rms_between: a branch without its gain or with short rows");
+  if (out && (!gain_next || ldo < d)) JLLM_FAIL("rms_between: an output without its gain or with short rows");
+  if (vec && vec_dtype != JLLM_F32 && vec_dtype != JLLM_BF16) JLLM_FAIL("rms_between: unknown dtype code %d", vec_dtype);
+  BetweenArgs A{x, d, a, lda, a2, lda2, s1, s2, gain, eps, rows, vec, vec_dtype == JLLM_BF16, gain_next, eps_next, out, ldo};
+  const size_t ea = a_dtype == JLLM_F32 ? 16 : 8, eo = out_dtype == JLLM_F32 ? 16 : 8, ev = vec_dtype == JLLM_F32 ? 16 : 8;
+  const bool wide = d % 4 == 0 && pn_aligned(x, 16) && (!a || (pn_aligned(a, ea) && lda % 4 == 0 && pn_aligned(gain, 16))) &&
+                    (!a2 || (pn_aligned(a2, ea) && lda2 % 4 == 0)) && pn_aligned(rows, 16) && (!vec || pn_aligned(vec, ev)) &&
+                    (!out || (pn_aligned(out, eo) && ldo % 4 == 0 && pn_aligned(gain_next, 16)));
+#define PN_LAUNCH(V, G) rms_between_kernel<TA, TO, V, G><<<n, PN_THREADS, 0, stream>>>(A)
+  JLLM_DISPATCH_1(a_dtype, TA, {
+    JLLM_DISPATCH_1(out_dtype, TO, {
+      if (wide && d <= PN_THREADS * 4)
+        PN_LAUNCH(4, 1);
+      else if (wide && d <= PN_THREADS * 8)
+        PN_LAUNCH(4, 2);
+      else if (wide && d <= PN_THREADS * 16)
+        PN_LAUNCH(4, 4);
+      else if (wide)
+        PN_LAUNCH(4, 8);
+      else if (d <= PN_THREADS * 4)
+        PN_LAUNCH(1, 4);
+      else if (d <= PN_THREADS * 16)
+        PN_LAUNCH(1, 16);
+      else
+        PN_LAUNCH(1, 32);
+    })
+  })
+#undef PN_LAUNCH
+  JLLM_CHECK_LAUNCH("rms_between");
+  return 0;
+}
 
 // a, a2 in a_dtype; gains, mu and state fp32. mu: with `state` [slots, d] and the rows' slots, one row per request
 extern "C" int jllm_rms_seam(float* x, int n, int d, const void* a, int lda, const void* a2, int lda2, int a_dtype, float s1,

@@ -81,9 +81,10 @@ def _declare(lib) -> None:
         "jllm_concat_rows": [_P, _P, _I, _I, _P, _I, _I, _P],
         "jllm_ssm_scan": [_P, _I, _P, _I, _I, _I, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P],
         "jllm_gated_group_norm": [_P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P, _I, _I, _I, _I, _F, _P],
-        "jllm_linear_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
-        "jllm_linear_chunks": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
+        "jllm_linear_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _P],
+        "jllm_linear_chunks": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _P, _P],
         "jllm_rms_seam": [_P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _P, _F, _P, _F, _P, _I, _I, _P, _P, _P, _P],
+        "jllm_rms_between": [_P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _F, _P, _P, _I, _P, _F, _P, _I, _I, _P],
         "jllm_token_shift": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
         "jllm_copy_page_rows": [_P, _I, _I, _I, _I, _L, _I, _I, _I, _P],
         "jllm_layernorm_seam": [_P, _P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _P, _P, _P, _P, _I, _F, _P, _I, _I, _P],
@@ -1603,24 +1604,33 @@ def linear_chunk_plan(segments):
     return requests, chunks
 
 
-def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers: torch.Tensor, state: torch.Tensor,
+def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers: Optional[torch.Tensor], state: torch.Tensor,
                      row_req: torch.Tensor, state_slots: torch.Tensor, n_requests: int, heads: int, dk: int, dv: int, *,
                      positions: Optional[torch.Tensor] = None, cos: Optional[torch.Tensor] = None,
                      sin: Optional[torch.Tensor] = None, rot_dims: int = 0, silu: bool = False, k_scale: float = 1.0,
-                     requests: Optional[torch.Tensor] = None, chunks: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """Linear attention with a fixed decay per head over the step's rows, request by request, from and into ``state``
+                     requests: Optional[torch.Tensor] = None, chunks: Optional[torch.Tensor] = None,
+                     decay_rows: Optional[torch.Tensor] = None, tau: float = 1.0) -> torch.Tensor:
+    """Linear attention with a decay over the step's rows, request by request, from and into ``state``
     [slots, heads, dv, dk] (fp32; a head's matrix S [dk, dv] column by column). ``y`` rows hold q and k (heads x dk) and v
     (heads x dv) at the given offsets; with ``silu`` all three pass silu; with ``rot_dims`` the pairs (i, i + rot_dims / 2)
     of every q and k head turn by the table rows of the positions; k is multiplied by ``k_scale``. Per head S <- d S + k
     v^T, o = S^T q with d from ``powers`` (``decay_powers``). Returns o, fp32 [T, heads x dv]. ``requests`` and ``chunks``
     (``linear_chunk_plan`` on the device): the chunked form on the matrix cores (fp32), where the sizes allow it; without
-    them the rows are walked one by one."""
-    _dev(y, powers, state, row_req, state_slots, positions, cos, sin, requests, chunks)
+    them the rows are walked one by one. ``decay_rows`` (fp32 [T, heads x dk], with ``powers`` None): a decay per key channel
+    and token instead, sigmoid(decay_rows)^(1 / tau), on the rows of S (no rotation)."""
+    _dev(y, powers, decay_rows, state, row_req, state_slots, positions, cos, sin, requests, chunks)
     _rows2d(y, "projection rows")
     T = y.shape[0]
     if min(q_off, k_off, v_off) < 0 or max(q_off + heads * dk, k_off + heads * dk, v_off + heads * dv) > y.shape[1]:
         raise KernelError("linear attention: q, k or v lie outside the projection rows")
-    if powers.dtype != torch.float32 or not powers.is_contiguous() or powers.shape != (heads, LINEAR_CHUNK + 1):
+    if (powers is None) == (decay_rows is None):
+        raise KernelError("linear attention: a decay per head or per channel")
+    if decay_rows is not None:
+        _rows2d(decay_rows, "decay rows")
+        if decay_rows.dtype != torch.float32 or decay_rows.shape != (T, heads * dk) or not tau > 0 or rot_dims:
+            raise KernelError(f"linear attention: {decay_rows.dtype} decay rows {tuple(decay_rows.shape)} for {(T, heads * dk)}, "
+                              f"tau {tau}, rotary width {rot_dims}")
+    elif powers.dtype != torch.float32 or not powers.is_contiguous() or powers.shape != (heads, LINEAR_CHUNK + 1):
         raise KernelError(f"linear attention: the decays' powers must be a contiguous fp32 [{heads}, {LINEAR_CHUNK + 1}] tensor")
     if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 4 or state.shape[1:] != (heads, dv, dk):
         raise KernelError(f"the state must be a contiguous fp32 [slots, {heads}, {dv}, {dk}] tensor")
@@ -1637,15 +1647,17 @@ def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers
     head = (_ptr(y), y.stride(0), int(q_off), int(k_off), int(v_off), _code(y.dtype), _ptr(positions) if rot_dims else None,
             _ptr(cos) if rot_dims else None, _ptr(sin) if rot_dims else None, int(rot_dims), 1 if silu else 0, float(k_scale),
             _ptr(powers), _ptr(state), _ptr(out), out.stride(0))
+    decay = (_ptr(decay_rows), decay_rows.stride(0) if decay_rows is not None else 0, 1.0 / float(tau))
     if requests is not None and chunks is not None and requests.numel() and chunks.numel():
         _i32(requests, 3 * n_requests, "requests of the chunk plan")
         _i32(chunks, 2, "chunks")
         n_chunks = chunks.numel() // 2
         before = torch.empty((n_chunks * heads * dv * dk,), dtype=torch.float32, device=y.device)
+        chunk_decay = torch.empty((n_chunks * heads * dk,), dtype=torch.float32, device=y.device) if decay_rows is not None else None
         if _try("jllm_linear_chunks", *head, _ptr(requests), _ptr(chunks), n_chunks, _ptr(before), _ptr(state_slots), T,
-                int(n_requests), heads, dk, dv, _stream()):
+                int(n_requests), heads, dk, dv, *decay, _ptr(chunk_decay), _stream()):
             return out
-    _call("jllm_linear_scan", *head, _ptr(row_req), _ptr(state_slots), T, int(n_requests), heads, dk, dv, _stream())
+    _call("jllm_linear_scan", *head, _ptr(row_req), _ptr(state_slots), T, int(n_requests), heads, dk, dv, *decay, _stream())
     return out
 
 
@@ -1706,6 +1718,46 @@ def rms_seam(residual: torch.Tensor, a: torch.Tensor, gain: torch.Tensor, eps: f
           float(scales[0]), float(scales[1]), _ptr(g1), _ptr(g2), float(branch_eps), _ptr(gain), float(eps), _ptr(out),
           out.stride(0) if out is not None else 0, _code(out.dtype) if out is not None else F32, _ptr(shift), _ptr(state),
           _ptr(state_slots), _stream())
+    return out
+
+
+def rms_between(residual: torch.Tensor, a: Optional[torch.Tensor] = None, gain: Optional[torch.Tensor] = None, eps: float = 0.0, *,
+                a2: Optional[torch.Tensor] = None, s1: float = 1.0, s2: float = 0.0, add_rows: Optional[torch.Tensor] = None,
+                add_vec: Optional[torch.Tensor] = None, nxt=None) -> Optional[torch.Tensor]:
+    """What happens to the fp32 residual rows between two sublayers that are normed on both sides, in one launch, each part
+    optional and in this order: ``residual += rms(s1 * a (+ s2 * a2)) * gain``; ``residual += add_rows`` (fp32, of its
+    shape); ``residual += add_vec`` ([width]); and rms(residual) * g' as a new tensor, which is returned: ``nxt`` is (g', its
+    eps, the new tensor's type). Gains are fp32."""
+    _dev(residual, a, a2, gain, add_rows, add_vec)
+    _residual2d(residual)
+    n, d = residual.shape
+    for t in (a, a2):
+        if t is not None:
+            _rows2d(t, "a sublayer's output")
+            if t.shape != (n, d):
+                raise KernelError(f"rms_between: a sublayer's output is {tuple(t.shape)}, the residual {(n, d)}")
+    if (a is None) != (gain is None) or (a is None and a2 is not None):
+        raise KernelError("rms_between: a sublayer's output and its norm come together")
+    if gain is not None:
+        _vec32(gain, d, "the norm's gain")
+    if a2 is not None and a2.dtype != a.dtype:
+        raise KernelError("rms_between: both branches must share a type")
+    if add_rows is not None and (add_rows.dtype != torch.float32 or add_rows.shape != (n, d) or not add_rows.is_contiguous()):
+        raise KernelError(f"rms_between: the further rows must be a contiguous fp32 {(n, d)} tensor")
+    if add_vec is not None and (add_vec.numel() != d or not add_vec.is_contiguous()):
+        raise KernelError(f"rms_between: the vector has {add_vec.numel()} entries, the rows have {d}")
+    out = None
+    if nxt is not None:
+        _dev(nxt[0])
+        _vec32(nxt[0], d, "the next norm's gain")
+        out = activation_rows(n, d, nxt[2], residual.device)
+    if n == 0:
+        return out
+    _call("jllm_rms_between", _ptr(residual), n, d, _ptr(a), a.stride(0) if a is not None else 0, _ptr(a2),
+          a2.stride(0) if a2 is not None else 0, _code(a.dtype) if a is not None else F32, float(s1), float(s2), _ptr(gain),
+          float(eps), _ptr(add_rows), _ptr(add_vec), _code(add_vec.dtype) if add_vec is not None else F32,
+          _ptr(nxt[0]) if nxt else None, float(nxt[1]) if nxt else 0.0, _ptr(out), out.stride(0) if out is not None else 0,
+          _code(out.dtype) if out is not None else F32, _stream())
     return out
 
 

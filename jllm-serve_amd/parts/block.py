@@ -99,12 +99,13 @@ def sublayer_output(part, xb, step, slot, width):
 
 class SandwichBlock(Part):
     """A norm in front of and behind each sublayer: x += norm_mixer_out(mixer(norm_in(x))); x += norm_ffn_out(ffn(
-    norm_post(x))). Where the norm part offers a ``seam`` (parts/norm.py: LayerNorm), the norm of a sublayer's output,
-    its add into the stream, a vector that joins the stream before the next layer, and the next sublayer's input norm
-    are one launch, handed on as the next block's input."""
+    norm_post(x))). A factor per channel behind an output norm (``mixer_scale_name`` / ``ffn_scale_name``) is taken into that
+    norm's gain when the weights are loaded. Where the norm part offers a ``seam`` (parts/norm.py), the norm of a
+    sublayer's output, its add into the stream, what else joins the stream before the next layer (the embedding output, a
+    vector), and the next sublayer's input norm are one launch, handed on as the next block's input."""
 
     chains_norms = True
-    takes_stream_vector = True  # forward(..., add_after=) adds that vector to the stream as its last act
+    takes_stream_vector = True  # forward(..., add_after=, add_rows_after=) adds that vector, those rows to the stream as its last act
 
     def __init__(self, spec, prefix, build, positions):
         ending = getattr(spec, "name_ending", ".weight")
@@ -129,13 +130,25 @@ class SandwichBlock(Part):
             self.ffn = part_factory("ffn", spec.ffn.kind)(spec.ffn, prefix, build)
             self.parts = (self.norm_in, self.mixer, self.norm_mixer_out, self.norm_post, self.ffn, self.norm_ffn_out)
         self.capturable = all(getattr(p, "capturable", True) for p in self.parts)
+        # output norms whose result is multiplied by a factor per channel
+        self.scales = [(f"{prefix}.{name}{ending}", part) for name, part in
+                       ((getattr(spec, "mixer_scale_name", ""), self.norm_mixer_out), (getattr(spec, "ffn_scale_name", ""), self.norm_ffn_out))
+                       if name and part is not None]
+        # a layer without a feed-forward that nevertheless names the factors behind one: its checkpoint may carry that
+        # sublayer's vectors all the same (they are not used)
+        self.unused = []
+        if self.ffn is None and getattr(spec, "ffn_scale_name", ""):
+            self.unused = [f"{prefix}.{n}{ending}" for n in (spec.norm_post_name, spec.norm_ffn_out_name, spec.ffn_scale_name) if n]
 
     def weight_specs(self):
-        return [w for p in self.parts for w in p.weight_specs()]
+        out = [w for p in self.parts for w in p.weight_specs()] + [WeightSpec(n, (self.width,), init="gain") for n, _ in self.scales]
+        return out + [WeightSpec(n, (self.width,), optional=True) for n in self.unused]
 
     def load(self, get):
         for p in self.parts:
             p.load(get)
+        for name, norm in self.scales:
+            norm.scale_channels(get(name))
 
     def cache_spec(self):
         return self.mixer.cache_spec()
@@ -147,36 +160,43 @@ class SandwichBlock(Part):
         return [pl for p in self.parts for pl in (p.step_planners() if hasattr(p, "step_planners") else [])]
 
     @staticmethod
-    def _join(norm, x, branch, add_vec, then):
-        """x += norm(branch) (+ add_vec); returns then's norm of the new x, or None when nobody prepared it."""
-        if hasattr(norm, "seam") and (then is None or hasattr(then, "seam")):
-            return norm.seam(x, [branch], [1.0], add_vec=add_vec, then=then)
+    def _seams(norm, then, add_rows):
+        """Whether ``norm`` does all of this in its own launch."""
+        return hasattr(norm, "seam") and (then is None or hasattr(then, "seam")) \
+            and (add_rows is None or getattr(norm, "seam_adds_rows", False))
+
+    def _join(self, norm, x, branch, add_rows, add_vec, then):
+        """x += norm(branch) (+ add_rows) (+ add_vec); returns then's norm of the new x, or None when nobody prepared it."""
+        if self._seams(norm, then, add_rows):
+            more = {"add_rows": add_rows} if add_rows is not None else {}
+            return norm.seam(x, [branch], [1.0], add_vec=add_vec, then=then, **more)
         x += norm.forward(branch).float()
+        if add_rows is not None:
+            x += add_rows
         if add_vec is not None:
             x += add_vec.float()
         return None
 
-    def forward(self, x, step, slot, normed_in=None, next_norm=None, add_after=None):
+    def forward(self, x, step, slot, normed_in=None, next_norm=None, add_after=None, add_rows_after=None):
         """``normed_in``: norm_in of x as the block before left it (a tensor) or None; ``next_norm``: the norm part that
-        reads x next; ``add_after``: a vector that joins the stream behind this layer. Returns ``next_norm`` of the new
-        x when the last seam prepared it."""
+        reads x next; ``add_after``: a vector that joins the stream behind this layer, ``add_rows_after``: rows that join
+        it before that. Returns ``next_norm`` of the new x when the last seam prepared it."""
         xb = normed_in if isinstance(normed_in, torch.Tensor) else self.norm_in.forward(x)
-        then, vec = (next_norm, add_after) if self.ffn is None else (self.norm_post, None)
+        then, rows, vec = (next_norm, add_rows_after, add_after) if self.ffn is None else (self.norm_post, None, None)
         scales = getattr(getattr(self.mixer, "spec", None), "scales", ())
         if hasattr(self.mixer, "outputs") and not getattr(self.mixer, "fused", False) and len(scales) == 2 \
-                and not getattr(self.mixer, "out_names", None) \
-                and hasattr(self.norm_mixer_out, "seam") \
-                and (then is None or hasattr(then, "seam")):
+                and not getattr(self.mixer, "out_names", None) and self._seams(self.norm_mixer_out, then, rows):
             # two weighted branches: their sum is taken inside the seam's launch
-            xb = self.norm_mixer_out.seam(x, self.mixer.outputs(xb, step, slot), list(scales), add_vec=vec, then=then)
+            more = {"add_rows": rows} if rows is not None else {}
+            xb = self.norm_mixer_out.seam(x, self.mixer.outputs(xb, step, slot), list(scales), add_vec=vec, then=then, **more)
         else:
-            xb = self._join(self.norm_mixer_out, x, sublayer_output(self.mixer, xb, step, slot, self.width), vec, then)
+            xb = self._join(self.norm_mixer_out, x, sublayer_output(self.mixer, xb, step, slot, self.width), rows, vec, then)
         if self.ffn is None:
             return xb
         if xb is None:
             xb = self.norm_post.forward(x)
         branch = sublayer_output(self.ffn, xb, step, None, self.width)
-        return self._join(self.norm_ffn_out, x, branch, add_after, next_norm)
+        return self._join(self.norm_ffn_out, x, branch, add_rows_after, add_after, next_norm)
 
 
 register_part("arrangement", "sandwich", SandwichBlock, replace=True)

@@ -1,9 +1,10 @@
-"""Linear attention with a fixed decay per head (config/schema.py: LinearAttentionSpec): a recurrent mixer whose
+"""Linear attention with a decay per head, or per key channel and token (config/schema.py: LinearAttentionSpec): a recurrent mixer whose
 per-request state has a fixed size, one matrix S [dim, vdim] per head in fp32 (kept column by column, [vdim, dim]) in the
 cache manager's state slots. Nothing is paged and nothing grows with the context.
 
 A step is
-  1. one product with the stacked weight [W_q | W_k | W_v | W_g],
+  1. one product with the stacked weight [W_q | W_k | W_v | W_g] (and, where the token chooses its decays, the narrow W_down
+     of their input, whose second half is a product of its own into fp32 rows),
   2. the recurrence over each request's rows in order, with the activation, the rotation and k's constant inside
      (``ops.linear_attention``; its read-out comes back raw, in fp32): row by row for steps of few rows per request, in
      chunks of 64 rows as fp32 matrix products for portions of prompts,
@@ -38,12 +39,18 @@ class LinearStepPlanner:
 
 class LinearAttention(Part):
     def __init__(self, spec: LinearAttentionSpec, prefix: str, build: BuildContext, positions):
-        if len(spec.decay) != spec.heads:
-            raise ValueError(f"{prefix}: {len(spec.decay)} decays for {spec.heads} heads")
+        if spec.decay_per not in ("head", "channel"):
+            raise ValueError(f"{prefix}: a decay per '{spec.decay_per}' is not built ('head' and 'channel' are)")
+        self.channel = spec.decay_per == "channel"
+        if len(spec.decay) != (0 if self.channel else spec.heads):
+            raise ValueError(f"{prefix}: {len(spec.decay)} fixed decays for {spec.heads} heads with a decay per {spec.decay_per}")
+        if self.channel and (not spec.tau > 0 or spec.decay_rank == 0 or spec.position is not None):
+            raise ValueError(f"{prefix}: a decay per key channel takes its input through a narrow middle ({spec.decay_rank}), with a "
+                             f"positive tau ({spec.tau}) and without a rotation")
         if spec.activation not in (None, "silu"):
             raise ValueError(f"{prefix}: activation '{spec.activation}' in front of the recurrence (silu is built)")
-        if spec.norm not in ("head", "whole"):
-            raise ValueError(f"{prefix}: norm '{spec.norm}' of the read-out ('head' and 'whole' are built)")
+        if spec.norm not in ("head", "head_gain", "whole"):
+            raise ValueError(f"{prefix}: norm '{spec.norm}' of the read-out ('head', 'head_gain' and 'whole' are built)")
         if spec.gate_fn not in ops.HEAD_GATES:
             raise ValueError(f"{prefix}: gate function '{spec.gate_fn}' ({sorted(ops.HEAD_GATES)} are built)")
         self.spec = spec
@@ -59,7 +66,8 @@ class LinearAttention(Part):
             raise ValueError(f"{prefix}: {e}") from None
         self.qk_dim = spec.heads * spec.dim
         self.v_dim = spec.heads * spec.vdim
-        self.w_in = self.w_o = self.gain = self.powers = None
+        self.decay_at = 2 * self.qk_dim + 2 * self.v_dim  # the stacked product's columns behind q | k | v | gate
+        self.w_in = self.w_o = self.gain = self.powers = self.w_decay_up = self.b_decay = None
 
     def _name(self, which: str) -> str:
         return f"{self.prefix}.{getattr(self.spec.names, which)}"
@@ -69,18 +77,29 @@ class LinearAttention(Part):
         out = [WeightSpec(self._name("q"), (self.qk_dim, d)), WeightSpec(self._name("k"), (self.qk_dim, d)),
                WeightSpec(self._name("v"), (self.v_dim, d)), WeightSpec(self._name("gate"), (self.v_dim, d)),
                WeightSpec(self._name("o"), (d, self.v_dim))]
-        if self.spec.norm == "whole":
-            out.append(WeightSpec(self._name("norm"), (self.v_dim,), init="gain"))
+        if self.spec.norm != "head":
+            out.append(WeightSpec(self._name("norm"), (self.v_dim if self.spec.norm == "whole" else self.spec.vdim,), init="gain"))
+        if self.channel:
+            r = self.spec.decay_rank
+            out += [WeightSpec(self._name("decay_down"), (r, d)), WeightSpec(self._name("decay_up"), (self.qk_dim, r)),
+                    WeightSpec(self._name("decay_bias"), (self.qk_dim,), init="bias")]
         return out
 
     def load(self, get):
-        stack = [get(self._name(n)) for n in ("q", "k", "v", "gate")]
+        stack = [get(self._name(n)) for n in ("q", "k", "v", "gate") + (("decay_down",) if self.channel else ())]
+        if self.channel:
+            self.w_decay_up = get(self._name("decay_up"))
+            self.b_decay = get(self._name("decay_bias")).float().contiguous()
+            if self.w_decay_up.shape[1] != stack[-1].shape[0]:
+                raise ValueError(f"{self.prefix}: the two halves of the decay's input disagree about their middle: "
+                                 f"{stack[-1].shape[0]} and {self.w_decay_up.shape[1]}")
         dt = stack[0].dtype if all(t.dtype == stack[0].dtype for t in stack) else torch.float32
         self.w_in = pad_rows(torch.cat([t.to(dt) for t in stack], dim=0).contiguous())
         self.w_o = get(self._name("o"))
-        if self.spec.norm == "whole":
+        if self.spec.norm != "head":
             self.gain = get(self._name("norm"))
-        self.powers = ops.decay_powers(self.spec.decay, self.build.device)
+        if not self.channel:
+            self.powers = ops.decay_powers(self.spec.decay, self.build.device)
 
     def state_spec(self):
         s = self.spec
@@ -112,13 +131,18 @@ class LinearAttention(Part):
         plan = step.plans.get(LinearStepPlanner.key)
         requests = plan.arrays.get("requests") if plan is not None else None
         chunks = plan.arrays.get("chunks") if plan is not None else None
+        decay_rows = None
+        if self.channel:  # what enters the recurrence besides the projections is fp32
+            decay_rows = ops.gemm(y[:, self.decay_at:self.decay_at + self.w_decay_up.shape[1]], self.w_decay_up, bias=self.b_decay,
+                                  out_dtype=torch.float32, exact=self.build.exact)
         o = ops.linear_attention(y, 0, self.qk_dim, 2 * self.qk_dim, self.powers, slot.state, step.row_req, step.state_slots,
                                  step.n_requests, s.heads, s.dim, s.vdim, positions=step.positions, cos=cos, sin=sin,
-                                 rot_dims=rdims, silu=s.activation == "silu", k_scale=s.k_scale, requests=requests, chunks=chunks)
+                                 rot_dims=rdims, silu=s.activation == "silu", k_scale=s.k_scale, requests=requests, chunks=chunks,
+                                 decay_rows=decay_rows, tau=s.tau)
         gate_at = 2 * self.qk_dim + self.v_dim
         gate = y[:, gate_at:gate_at + self.v_dim]
-        if s.norm == "head":
-            return ops.heads_finish(o, s.heads, 1, s.vdim, self.build.dtype, normed=True, eps=s.eps, gate=gate,
+        if s.norm != "whole":
+            return ops.heads_finish(o, s.heads, 1, s.vdim, self.build.dtype, normed=True, eps=s.eps, gain=self.gain, gate=gate,
                                     gate_fn=s.gate_fn, out=out, out_mul=out_mul)
         return ops.gated_group_norm(o, gate, self.gain, s.eps, 1, self.build.dtype, gate_fn=s.gate_fn, gate_last=True, out=out,
                                     out_mul=out_mul)

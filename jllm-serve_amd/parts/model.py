@@ -57,6 +57,7 @@ class DecoderModel:
         # matrices that mix the stream with the embedding output before a run (ScheduleEntry.mix_before), by tensor name
         self.stream_mix_names = sorted({e.mix_before.name for e in config.schedule if e.mix_before is not None})
         self.stream_mixes = {}
+        self.keeps_embedding = bool(self.stream_mix_names) or any(getattr(e, "add_embedding", False) for e in config.schedule)
         self.watch = None  # a function (run, x) called with the stream after every run (tests, debugging)
         # a part that walks the step's requests on the host sets ``capturable = False``; then decode steps are
         # never recorded as graphs
@@ -134,9 +135,9 @@ class DecoderModel:
             x = self.embed_norm.forward(x, out_dtype=torch.float32, copies=self.streams) if hasattr(self.embed_norm, "vectors") \
                 else self.embed_norm.forward(x).float()
         schedule = self.config.schedule
-        x0 = x.clone() if self.stream_mix_names else None  # the embedding output, for the runs that mix it back in
+        x0 = x.clone() if self.keeps_embedding else None  # the embedding output, for the runs that bring it back in
         carry = None  # the next block's input norm, when the block before prepared it (parts/block.py)
-        added = False  # this run's vector already joined the stream (the block before added it on its way out)
+        added = False  # what joins the stream before this run already did (the block before added it on its way out)
         for run, e in enumerate(schedule):
             layer = self.layers[e.layer]
             if e.mix_before is not None:
@@ -145,6 +146,9 @@ class DecoderModel:
                 x = ops.gemm(ops.concat_rows(x, x0, self.build.dtype), self.stream_mixes[e.mix_before.name], bias=vec,
                              out=torch.empty_like(x), exact=self.build.exact)
                 added = True
+                carry = None
+            if e.add_embedding and not added:
+                ops.rms_between(x, add_rows=x0)
                 carry = None
             if e.add_before is not None and not added:
                 ops.layernorm_seam(x, 0.0, add_vec=self._stream_vector(e.add_before))
@@ -159,13 +163,14 @@ class DecoderModel:
                 next_norm = None
                 if getattr(nxt, "chains_norms", False):  # a reader may need the state of the run it reads for
                     next_norm = nxt.stream_reader(slots[run + 1]) if hasattr(nxt, "stream_reader") else getattr(nxt, "norm_in", None)
-                if nxt_e is not None and nxt_e.add_before is not None and nxt_e.mix_before is None and self.watch is None \
-                        and getattr(layer, "takes_stream_vector", False):
+                joins = nxt_e is not None and (nxt_e.add_before is not None or nxt_e.add_embedding)
+                if joins and nxt_e.mix_before is None and self.watch is None and getattr(layer, "takes_stream_vector", False):
                     carry = layer.forward(x, step, slots[run], normed_in=carry, next_norm=next_norm,
-                                          add_after=self._stream_vector(nxt_e.add_before))
+                                          add_after=self._stream_vector(nxt_e.add_before) if nxt_e.add_before is not None else None,
+                                          add_rows_after=x0 if nxt_e.add_embedding else None)
                     added = True
                 else:
-                    if nxt_e is not None and (nxt_e.add_before is not None or nxt_e.mix_before is not None):
+                    if joins or (nxt_e is not None and nxt_e.mix_before is not None):
                         next_norm = None  # the stream changes before the next block reads it
                     carry = layer.forward(x, step, slots[run], normed_in=carry, next_norm=next_norm)
             if self.watch is not None:  # (with several streams: their sum)

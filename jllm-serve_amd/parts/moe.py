@@ -95,7 +95,7 @@ register_part("ffn", "table_moe", TableMoe, replace=True)
 class RoutedMoe(Part):
     """A mixture of experts chosen by a router: x += sum over the row's chosen experts of weight * expert(xb).
 
-    The router's logits are an fp32 product of the rows with the router's weight (held in fp32); ``ops.moe_router`` turns
+    The router's logits are an fp32 product of the rows with the router's weight (and a bias, where it has one); ``ops.moe_router`` turns
     them into the chosen experts and their weights per row (sigmoid or softmax scores, a correction on the choice,
     groups of experts of which only the best are open, weights normalised over the chosen or not). A shared expert
     (``spec.shared``) runs for every row; with ``spec.shared_gate`` its fp32 rows are multiplied by the sigmoid of one
@@ -119,7 +119,7 @@ class RoutedMoe(Part):
         self.limit = float(getattr(spec, "limit", 0.0))
         self.takes_normed_rows = False
         self.shared = part_factory("ffn", spec.shared.kind)(spec.shared, prefix, build) if spec.shared is not None else None
-        self.w_gate = self.w_up = self.w_down = self.w_router = self.correction = None
+        self.w_gate = self.w_up = self.w_down = self.w_router = self.b_router = self.correction = None
 
     def _expert(self, e: int, which: str) -> str:
         n = self.spec.names
@@ -135,6 +135,8 @@ class RoutedMoe(Part):
             out += [WeightSpec(self._expert(e, "gate"), (s.hidden, d)), WeightSpec(self._expert(e, "up"), (s.hidden, d)),
                     WeightSpec(self._expert(e, "down"), (d, s.hidden))]
         out.append(WeightSpec(self._own("router"), (s.experts, d)))
+        if s.router_bias:
+            out.append(WeightSpec(self._own("router_bias"), (s.experts,), init="bias"))
         if s.correction:
             out.append(WeightSpec(self._own("correction"), (s.experts,), init="bias"))
         if self.shared is not None:
@@ -157,6 +159,9 @@ class RoutedMoe(Part):
             self.shared.load(get)
         fast = w.dtype == torch.bfloat16 and self.build.dtype == torch.bfloat16 and not self.build.exact
         self.w_router = pad_rows(w) if fast else w.float().contiguous()
+        if s.router_bias:  # fp32, with zeros for the product's further rows
+            b = get(self._own("router_bias")).float()
+            self.b_router = torch.cat([b, torch.zeros(self.w_router.shape[0] - s.experts, dtype=b.dtype, device=b.device)]).contiguous()
         self.correction = get(self._own("correction")).float().contiguous() if s.correction else None
 
     def forward(self, xb, residual, step, then_norm=None):
@@ -174,7 +179,7 @@ class RoutedMoe(Part):
         s, exact = self.spec, self.build.exact
         T = xb.shape[0]
         # fp32 logits: plain FMAs for an fp32 router, the matrix cores' exact products for a bf16 one
-        zz = ops.gemm(xb, self.w_router, out_dtype=torch.float32, exact=self.w_router.dtype == torch.float32)
+        zz = ops.gemm(xb, self.w_router, bias=self.b_router, out_dtype=torch.float32, exact=self.w_router.dtype == torch.float32)
         z = zz[:, :s.experts]
         shared_rows = self.shared.output(xb, step) if self.shared is not None else None
         shared_gate = zz[:, s.experts] if s.shared_gate else None

@@ -18,7 +18,7 @@ class RMSNorm(Part):
         self.weight_name = weight_name
         self.out_dtype = build.dtype
         self.one_plus = bool(getattr(spec, "one_plus", False))
-        self.gain = None
+        self.gain = self.gain32 = None
 
     def weight_specs(self):
         return [WeightSpec(self.weight_name, (self.dim,), init="bias" if self.one_plus else "gain")]
@@ -27,6 +27,7 @@ class RMSNorm(Part):
         self.gain = get(self.weight_name)
         if self.one_plus:  # the stored weight lies around zero; in fp32, since 1 + w has more digits than a bf16 holds
             self.gain = (self.gain.float() + 1.0).contiguous()
+        self.gain32 = self.gain.float().contiguous()  # what the launches between two sublayers take
 
     def forward(self, x, rows=None):
         return ops.rmsnorm(x, self.gain, self.eps, self.out_dtype, rows)
@@ -38,7 +39,11 @@ class RMSNorm(Part):
     def scale_output(self, factor: float) -> None:
         """From now on the norm's output is ``factor`` times what it was (the gain in fp32)."""
         if factor != 1.0:
-            self.gain = (self.gain.float() * factor).contiguous()
+            self.gain = self.gain32 = (self.gain.float() * factor).contiguous()
+
+    def scale_channels(self, factors: torch.Tensor) -> None:
+        """The same with a factor per channel."""
+        self.gain = self.gain32 = (self.gain.float() * factors.float()).contiguous()
 
     def after_add(self, a, w, residual, bias=None, exact=False):
         """residual += a @ w.T (+ bias), and this norm of the result as a promise: the product that makes the new
@@ -49,10 +54,22 @@ class RMSNorm(Part):
         """``residual += this norm of a sublayer's output`` in one launch. ``branches``: the output, or two branches'
         outputs, each RMS-normed with its gain (``branch_gains``, ``branch_eps``), weighed and added first. ``then``: what
         the next reader wants of the new rows: keyword arguments of ``ops.rms_seam`` (its type, a token shift), or None."""
-        if self.gain.dtype != torch.float32:
-            self.gain = self.gain.float().contiguous()
-        return ops.rms_seam(residual, branches[0], self.gain, self.eps, a2=branches[1] if len(branches) == 2 else None,
+        return ops.rms_seam(residual, branches[0], self.gain32, self.eps, a2=branches[1] if len(branches) == 2 else None,
                             branch_gains=branch_gains, scales=scales, branch_eps=branch_eps, **(then or {}))
+
+    seam_adds_rows = True  # ``seam`` takes ``add_rows``
+
+    def seam(self, residual, branches, scales, add_vec=None, then=None, add_rows=None):
+        """The launch between two sublayers that are normed on both sides: ``residual += this norm of (sum_i scales[i] *
+        branches[i])`` (one or two branches); then ``residual += add_rows`` (fp32 rows), ``+= add_vec`` (a vector); returns
+        ``then``'s norm of the new rows (``then``: the norm part that reads them next, or None)."""
+        if not 1 <= len(branches) <= 2 or len(scales) != len(branches):
+            raise ValueError("the seam takes one or two branches with a scale each")
+        two = len(branches) == 2
+        nxt = (then.gain32, then.eps, then.out_dtype) if isinstance(then, RMSNorm) else None
+        out = ops.rms_between(residual, branches[0], self.gain32, self.eps, a2=branches[1] if two else None, s1=scales[0],
+                              s2=scales[1] if two else 0.0, add_rows=add_rows, add_vec=add_vec, nxt=nxt)
+        return then.forward(residual) if then is not None and nxt is None else out
 
 
 register_part("norm", "rmsnorm", RMSNorm, replace=True)
@@ -91,6 +108,11 @@ class LayerNorm(Part):
         if factor != 1.0:
             self.gain = (self.gain.float() * factor).contiguous()
             self.bias = (self.bias.float() * factor).contiguous()
+
+    def scale_channels(self, factors: torch.Tensor) -> None:
+        """The same with a factor per channel."""
+        self.gain = (self.gain.float() * factors.float()).contiguous()
+        self.bias = (self.bias.float() * factors.float()).contiguous()
 
     def forward(self, x, rows=None):
         return ops.layernorm_seam(x, self.eps, nxt=(self.gain, self.bias), out_dtype=self.out_dtype, rows=rows)

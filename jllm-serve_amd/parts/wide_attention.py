@@ -3,8 +3,8 @@ put around the softmax (config/schema.py: WideAttentionSpec): two score maps per
 (differential attention), a norm with gains over the whole q and k projections or over every head alone, rotation of
 neighbouring pairs or of the two halves of a head's rotated part, capped scores, a query scale that grows with the
 position, a factor per head on the scores, a distance penalty per head, a sliding window that may keep the first keys or
-chunks of the sequence, values that are the unnormed keys, a learned sink in the softmax's denominator, an output gate
-per channel or per head.
+chunks of the sequence, values that are the unnormed keys, a learned sink (or a plain one) in the softmax's denominator,
+an output gate per channel or per head.
 
 A step is
   1. one product with the stacked weight [W_q | W_k | W_v | W_g] and the stacked bias (zeros for the gate's rows),
@@ -53,7 +53,9 @@ class WideAttention(Part):
             raise ValueError(f"{prefix}: {spec.maps} score maps per head (one or two are built)")
         if spec.qk_norm not in (None, "whole", "head"):
             raise ValueError(f"{prefix}: q/k norm '{spec.qk_norm}' is not built for this mixer ('whole' and 'head' are)")
-        if spec.sink and spec.maps != 1:
+        if spec.sink and spec.unit_sink:
+            raise ValueError(f"{prefix}: a learned sink beside the one without a tensor")
+        if (spec.sink or spec.unit_sink) and spec.maps != 1:
             raise ValueError(f"{prefix}: a sink with {spec.maps} score maps per head")
         if spec.keep_first and not spec.window:
             raise ValueError(f"{prefix}: first keys are kept beside a window, and this mixer has none")
@@ -129,6 +131,8 @@ class WideAttention(Part):
             self.b_in = pad_rows(torch.cat(b).contiguous())
         if s.sink:
             self.sinks = get(self._name("sink")).float().contiguous()
+        if s.unit_sink:  # exp(0) in every denominator
+            self.sinks = torch.zeros(s.heads, dtype=torch.float32, device=self.build.device)
         if s.head_temp:  # rides on q: (temp q) . k
             self.temp = get(self._name("temp")).float().contiguous()
         if s.qk_norm in ("whole", "head"):
