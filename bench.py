@@ -28,6 +28,10 @@ Miforax model of the same width, heads, window and feed-forwards.
 `--workload compare --design gubotar [--size 2k|4k]` measures a Gubotar model (chunked attention beside linear attention
 with a fixed decay, and retention layers, in turn; norms behind the sublayers, a token shift in front of every mixer)
 beside the Kebepel model of the same width, heads and feed-forward.
+`--workload compare --design dazilix [--size 2k|4k]` measures a Dazilix model (chunked attention and linear attention with a
+decay per key channel and token, in turn; norms on both sides of every sublayer; router-chosen experts in every layer)
+beside the Gubotar model of the same width and heads whose dense feed-forward has the weights a token passes through,
+and the Pivipel model of the same width, heads and experts.
 `--workload compare [--size 2k|4k]` is another run altogether: a Miforax model (latent attention with a window, dense
 and table-routed expert layers in turn) beside the closest model the engine had before, a Qwen3 dense model with the
 same width, layers, heads, window and feed-forward width, both with random weights: prefill of 2,048 tokens and
@@ -519,6 +523,91 @@ def compare_gubotar(args) -> dict:
     return out
 
 
+DAZILIX_EXTRA = {  # what a Dazilix model has beyond the sizes it shares with the Miforax model of the same name
+    "2k": dict(g_heads=16, g_dim=128, g_vdim=128, tau=16.0, middle=16, rot_dims=64),
+    "4k": dict(g_heads=32, g_dim=128, g_vdim=128, tau=16.0, middle=16, rot_dims=64),
+}
+
+
+def dazilix_config(z: dict) -> dict:
+    """Attention in chunks as long as the measured prompts and linear attention with a decay per key channel in turn, routed
+    experts in every layer; no loop."""
+    att = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"], "scale": z["dim"] ** -0.5,
+           "mask": {"size": GUBOTAR_CHUNK}, "rot": {"base": 1e4, "dims": z["rot_dims"]}}
+    gla = {"heads": z["g_heads"], "dim": z["g_dim"], "vdim": z["g_vdim"], "tau": z["tau"]}
+    moe = {"kind": "moe", "router": {"experts": z["experts"], "top": z["top"]}, "expert": {"ff": z["expert_ff"]}}
+    return {"architecture": "Dazilix", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "max_positions": 8192,
+            "layers": [{"type": "gla" if i % 2 else "attention", "mixer": gla if i % 2 else att, "mlp": moe} for i in range(z["layers"])]}
+
+
+class DazilixWork:
+    """Bytes and flops of passes over a Dazilix model of the sizes ``z`` (the interface of ``Work``). A decode step reads
+    every weight outside the experts, of the experts at most batch x top per layer, per request the keys and values (cached
+    as two tensors) of its chunk, and reads and writes the recurrent matrices (fp32); a row costs 2 flops per weight it
+    passes through, per (row, key) pair and head 4 dim, and in a recurrence 4 dim vdim per head."""
+
+    def __init__(self, z: dict, dtype: str):
+        self.z = z
+        self.L, self.d, self.H, self.Hkv, self.F, self.V, self.hd = z["layers"], z["width"], z["heads"], z["kv_heads"], z["top"] * z["expert_ff"], z["vocab"], z["dim"]
+        self.esize = 2 if dtype == "bf16" else 4
+        self.dtype = dtype
+        d, dk = self.d, z["dim"]
+        n_gla = self.L // 2
+        n_att = self.L - n_gla
+        gh, gk, gv, mid = z["g_heads"], z["g_dim"], z["g_vdim"], z["middle"]
+        self.mixers = n_att * (2 * z["heads"] + z["kv_heads"]) * dk * d + n_gla * (gh * (2 * gk + 3 * gv) * d + mid * (d + gh * gk))
+        self.expert = 3 * d * z["expert_ff"]
+        self.router = z["experts"] * d
+        self.kv_bytes_per_token = n_att * z["kv_heads"] * 2 * dk * self.esize
+        matrices = n_gla * gh * gk * gv
+        self.state_bytes = matrices * 4 * 2
+        self.pair_flops = n_att * 4 * z["heads"] * dk
+        self.row_flops = 4 * matrices
+        self.weight_bytes = (self.mixers + self.L * (self.router + z["experts"] * self.expert) + self.V * d) * self.esize
+
+    def decode_bytes(self, tokens_held: float, batch: int = 0) -> float:
+        z = self.z
+        touched = min(z["experts"], max(batch, 1) * z["top"])
+        w = self.mixers + self.L * (self.router + touched * self.expert) + self.V * self.d
+        return w * self.esize + self.kv_bytes_per_token * min(tokens_held, GUBOTAR_CHUNK * max(batch, 1)) + self.state_bytes * max(batch, 1)
+
+    def pairs(self, T: int) -> float:
+        return sum(i % GUBOTAR_CHUNK + 1 for i in range(T))
+
+    def flops(self, rows: float, pairs: float, selected: float) -> float:
+        per_row = self.mixers + self.L * (self.router + self.z["top"] * self.expert)
+        return rows * (2.0 * per_row + self.row_flops) + self.pair_flops * pairs + 2.0 * self.V * self.d * selected
+
+
+def compare_dazilix(args) -> dict:
+    """``--workload compare --design dazilix``: the Dazilix model of ``--size``, the Gubotar model of the same width, heads
+    and weights per token, and the Pivipel model of the same width, heads and experts, one after the other: prefill of 2,048
+    tokens in one portion, decoding at batch 8 and 64 behind prompts of 1,152 tokens."""
+    z = {**COMPARE_SIZES[args.size], **DAZILIX_EXTRA[args.size], "window": GUBOTAR_CHUNK}
+    zg = dict(KEBEPEL_SIZES[args.size], ff=z["top"] * z["expert_ff"])
+    zp = {**z, **PIVIPEL_EXTRA[args.size]}
+    ctx = 4096
+    decodes = [dict(key=f"b{B}", batch=B, prompt_len=1152, steps=args.point_steps, warmup=4) for B in (8, 64)]
+    prefills = [dict(key="main", tokens=2048, portion=2048)]
+    out = {"metric": f"Dazilix beside Gubotar and Pivipel at equal sizes ({args.size})", "unit": "tok/s", "n_gpus": 1, "dtype": "bf16",
+           "data": "synthetic (random weights N(0,0.02), uniform-random token ids)", "higher_is_better": True,
+           "config": {"size": args.size, **z, "context": ctx, "page_size": PAGE}, "models": {}}
+    for name, shape, work in (("dazilix", dazilix_config(z), DazilixWork(z, "bf16")), ("gubotar", gubotar_config(zg), GubotarWork(zg, "bf16")),
+                              ("pivipel", pivipel_config(zp), PivipelWork(zp, "bf16"))):
+        r = steady(args, name, "bf16", 0, ctx, decodes, prefills, shape=shape, work=work)
+        m = {"prefill_2048_tok_s": r["prefill"]["main"]["value"], "prefill_2048_ms": r["prefill"]["main"]["ms"],
+             "prefill_flop_frac": r["prefill"]["main"]["frac"]}
+        for B in (8, 64):
+            s_, held, by = r["decode"][f"b{B}"]
+            m[f"decode_b{B}_tok_s"] = round(B / s_, 1)
+            m[f"decode_b{B}_ms"] = round(s_ * 1e3, 3)
+            m[f"decode_b{B}_hbm_frac"] = round(by / s_ / HBM_PEAK, 4)
+        out["models"][name] = m
+    out["value"] = out["models"]["dazilix"]["decode_b8_tok_s"]
+    return out
+
+
 def compare_workload(args) -> dict:
     """``--workload compare``: the Miforax model of ``--size`` and the Qwen3 dense model of the same sizes, one after
     the other: prefill of 2,048 tokens in one portion, decoding at batch 8 and 64 with every window full."""
@@ -666,9 +755,10 @@ def main() -> int:
                     help="steady: timed decode steps at a fixed batch (the default run); serve: a request set run to the end; "
                          "compare: a Miforax model beside the Qwen3 dense model of the same sizes")
     ap.add_argument("--size", default="2k", choices=sorted(COMPARE_SIZES), help="compare: which sizes")
-    ap.add_argument("--design", default="miforax", choices=["miforax", "kebepel", "ratasun", "pivipel", "gubotar"],
+    ap.add_argument("--design", default="miforax", choices=["miforax", "kebepel", "ratasun", "pivipel", "gubotar", "dazilix"],
                     help="compare: which design stands beside the Qwen3 dense model of the same sizes (ratasun and pivipel: "
-                         "beside the Miforax model of the same sizes; gubotar: beside the Kebepel model)")
+                         "beside the Miforax model of the same sizes; gubotar: beside the Kebepel model; dazilix: beside the "
+                         "Gubotar and the Pivipel model)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
@@ -678,7 +768,8 @@ def main() -> int:
         print(json.dumps(serve_workload(args)))
         return 0
     if args.workload == "compare":
-        run = {"kebepel": compare_kebepel, "ratasun": compare_ratasun, "pivipel": compare_pivipel, "gubotar": compare_gubotar}.get(args.design, compare_workload)
+        run = {"kebepel": compare_kebepel, "ratasun": compare_ratasun, "pivipel": compare_pivipel, "gubotar": compare_gubotar,
+               "dazilix": compare_dazilix}.get(args.design, compare_workload)
         print(json.dumps(run(args)))
         return 0
 

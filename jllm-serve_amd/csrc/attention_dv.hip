@@ -111,6 +111,134 @@ __global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_kernel(
   }
 }
 
+// The same with the norm over the whole of q and the whole of k, for rows of few enough entries whose sizes are multiples
+// of V (16 bytes of T): a thread keeps its entries in registers, everything a row needs is requested before the first sum,
+// both sums share a barrier, and the heads pass through LDS once, for the other side of a rotated pair.
+template <typename T>
+__device__ __forceinline__ void prep_load(const T* p, float (&v)[16 / sizeof(T)]) {
+  if constexpr (sizeof(T) == 2) {
+    const uint4 u = *(const uint4*)p;
+    const uint32_t w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[2 * e] = __uint_as_float(w[e] << 16), v[2 * e + 1] = __uint_as_float(w[e] & 0xffff0000u);
+  } else {
+    const float4 u = *(const float4*)p;
+    v[0] = u.x, v[1] = u.y, v[2] = u.z, v[3] = u.w;
+  }
+}
+template <typename T>
+__device__ __forceinline__ void prep_store(T* p, const float (&v)[16 / sizeof(T)]) {
+  if constexpr (sizeof(T) == 2) {
+    uint32_t w[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[e] = (uint32_t)f32_to_bf16(v[2 * e]).bits | ((uint32_t)f32_to_bf16(v[2 * e + 1]).bits << 16);
+    *(uint4*)p = uint4{w[0], w[1], w[2], w[3]};
+  } else {
+    *(float4*)p = float4{v[0], v[1], v[2], v[3]};
+  }
+}
+
+template <typename T, typename TG, int G>
+__global__ __launch_bounds__(PREP_THREADS) void qkv_prepare_whole_kernel(
+    T* __restrict__ qkv, int ld, const int* __restrict__ positions, const int* __restrict__ slots, int q_slots, int k_slots,
+    int v_heads, int dk, int dv, const TG* __restrict__ gq, const TG* __restrict__ gk, float eps,
+    const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot_dims, float temp_coef, int temp_every,
+    T* __restrict__ kcache, T* __restrict__ vcache, int page_size, int pair_halves, const float* __restrict__ head_mul, int maps,
+    int tied) {
+  constexpr int V = 16 / sizeof(T);
+  extern __shared__ __align__(16) float sm[];
+  __shared__ float red[2][PREP_THREADS / 64];
+  const int t = blockIdx.x;
+  const int nq = q_slots * dk, n = nq + k_slots * dk, half = rot_dims >> 1;
+  T* row = qkv + (size_t)t * ld;
+  const int pos = positions[t];
+  const int slot = slots ? slots[t] : -1;
+  float x[G][V], gn[G][V], c[G][V], s[G][V];
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = min((int)(threadIdx.x + k * PREP_THREADS) * V, n - V);
+    prep_load(row + i, x[k]);
+    const TG* g = i < nq ? gq + i : gk + (i - nq);
+#pragma unroll
+    for (int e = 0; e < V; ++e) gn[k][e] = ldf(g, e);
+  }
+#pragma unroll
+  for (int k = 0; k < G; ++k) {  // the table's entries of a group: V neighbours, or with neighbouring pairs V / 2
+    const int e0 = (int)(threadIdx.x + k * PREP_THREADS) * V % dk;
+    const int f = e0 >= rot_dims ? 0 : pair_halves ? (e0 < half ? e0 : e0 - half) : e0 >> 1;
+    const size_t at = (size_t)pos * half + f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const size_t j = at + (pair_halves ? e : e >> 1);
+      c[k][e] = rot_dims ? cos_t[j] : 1.f;
+      s[k][e] = rot_dims ? sin_t[j] : 0.f;
+    }
+  }
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PREP_THREADS) * V;
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss = fmaf(x[k][e], x[k][e], ss);
+    sq += i < nq ? ss : 0.f;
+    sk += i >= nq && i < n ? ss : 0.f;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) red[0][threadIdx.x >> 6] = sq, red[1][threadIdx.x >> 6] = sk;
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int w = 0; w < PREP_THREADS / 64; ++w) sq += red[0][w], sk += red[1][w];
+  const float rq = norm_scale(sq, nq, eps), rk = norm_scale(sk, n - nq, eps);
+  const bool stores = slot >= 0;
+  const int page = stores ? slot / page_size : 0, off = stores ? slot % page_size : 0;
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PREP_THREADS) * V;
+    if (i >= n) continue;
+    if (tied && stores && i >= nq)  // the values are the k columns as they came
+      prep_store(vcache + (((size_t)page * k_slots + (i - nq) / dk) * page_size + off) * dk + (i - nq) % dk, x[k]);
+    const float r = i < nq ? rq : rk;
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[k][e] = x[k][e] * r * gn[k][e];
+    if (rot_dims && pair_halves && i % dk < rot_dims)
+#pragma unroll
+      for (int e = 0; e < V; ++e) sm[i + e] = x[k][e];
+  }
+  if (rot_dims && pair_halves) __syncthreads();
+  float temp = 1.0f;
+  if (temp_every > 0) temp = 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f);
+#pragma unroll
+  for (int k = 0; k < G; ++k) {
+    const int i = (threadIdx.x + k * PREP_THREADS) * V;
+    if (i >= n) continue;
+    const int e0 = i % dk;
+    if (e0 < rot_dims) {
+      float o[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) o[e] = pair_halves ? sm[i + e + (e0 < half ? half : -half)] : x[k][e ^ 1];
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const bool first = pair_halves ? e0 < half : !(e & 1);
+        x[k][e] = first ? x[k][e] * c[k][e] - o[e] * s[k][e] : x[k][e] * c[k][e] + o[e] * s[k][e];
+      }
+    }
+    if (i < nq) {
+      const float mul = head_mul ? temp * head_mul[i / dk / maps] : temp;
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[k][e] *= mul;
+      prep_store(row + i, x[k]);
+    } else if (stores) {
+      prep_store(kcache + (((size_t)page * k_slots + (i - nq) / dk) * page_size + off) * dk + e0, x[k]);
+    }
+  }
+  if (tied || !stores) return;
+  for (int i = threadIdx.x * V; i < v_heads * dv; i += PREP_THREADS * V)
+    *(uint4*)(vcache + (((size_t)page * v_heads + i / dv) * page_size + off) * dv + i % dv) = *(const uint4*)(row + n + i);
+}
+
 extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, const int* positions, const int* slots,
                                 int q_slots, int k_slots, int v_heads, int dk, int dv, const void* gq, const void* gk,
                                 int gain_dtype, float eps, const float* cos_t, const float* sin_t, int rot_dims,
@@ -125,6 +253,31 @@ extern "C" int jllm_qkv_prepare(void* qkv, int ld, int dtype, int n_tokens, cons
   if ((gq == nullptr) != (gk == nullptr)) JLLM_FAIL("qkv_prepare: the norm takes gains for both q and k");
   if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims && (!cos_t || !sin_t))) JLLM_FAIL("qkv_prepare: a rotary width of %d for heads of %d", rot_dims, dk);
   if (page_size <= 0) JLLM_FAIL("qkv_prepare: page_size %d", page_size);
+  const int V = dtype == JLLM_F32 ? 4 : 8, n_qk = (q_slots + k_slots) * dk;
+  if (gq && !norm_per_head && (dtype == JLLM_F32 || dtype == JLLM_BF16) && n_qk <= PREP_THREADS * V * 4 && dk % V == 0 && (tied_values || dv % V == 0) &&
+      ld % V == 0 && rot_dims % (pair_halves ? 2 * V : V) == 0 && ((uintptr_t)qkv & 15) == 0 && ((uintptr_t)kcache & 15) == 0 && ((uintptr_t)vcache & 15) == 0) {
+    const int per = (n_qk + PREP_THREADS * V - 1) / (PREP_THREADS * V);
+    const size_t lds = rot_dims && pair_halves ? (size_t)n_qk * sizeof(float) : 0;
+    if (lds <= 64 * 1024 - 64) {
+#define PREP_WHOLE(G)                                                                                                          \
+  qkv_prepare_whole_kernel<T, TG, G><<<n_tokens, PREP_THREADS, lds, stream>>>(                                                 \
+      (T*)qkv, ld, positions, slots, q_slots, k_slots, v_heads, dk, dv, (const TG*)gq, (const TG*)gk, eps, cos_t, sin_t, rot_dims, \
+      temp_coef, temp_every, (T*)kcache, (T*)vcache, page_size, pair_halves, head_mul, maps, tied_values)
+      JLLM_DISPATCH_1(dtype, T, {
+        JLLM_DISPATCH_1(gain_dtype, TG, {
+          if (per <= 1)
+            PREP_WHOLE(1);
+          else if (per <= 2)
+            PREP_WHOLE(2);
+          else
+            PREP_WHOLE(4);
+        })
+      })
+#undef PREP_WHOLE
+      JLLM_CHECK_LAUNCH("qkv_prepare");
+      return 0;
+    }
+  }
   // with few rows four heads per workgroup (a wave each) where nothing spans a whole projection: a row is a chain of waits,
   // which is then shared out over several workgroups
   int parts = (gq && !norm_per_head) ? 1 : (q_slots + k_slots + PREP_THREADS / 64 - 1) / (PREP_THREADS / 64);

@@ -1,6 +1,7 @@
 // Linear attention with a decay: S <- D S + k v^T, o = S^T q with S [dk, dv] per head, no softmax and no denominator. D is
 // one fixed number per head, or (channel decay) one number per head, key channel and token that acts on the rows of S:
-// alpha = sigmoid(z)^(1 / tau) with z an fp32 product's rows. fp32 or bf16 projections, everything from there on and the state in fp32. q, k and v are columns of one
+// alpha = sigmoid(z)^(1 / tau) with z = W_up m + bias for a narrow row m that is columns of the projection's rows too. z is
+// computed where it is used (in fp32), which is cheaper than a launch that writes its rows. fp32 or bf16 projections, everything from there on and the state in fp32. q, k and v are columns of one
 // projection's rows; on their way in they pass, as asked, silu (all three), a rotation of the pairs (i, i + rot / 2) among
 // the first rot entries of every q and k head by the row's position, and a constant on k. A request's rows of a step are
 // consecutive and in order (row_req ascends), their positions too.
@@ -37,14 +38,14 @@
 #include <math.h>
 
 #include "common.h"
+#include "mfma.h"
 #include "recurrence.h"
 
 #define LIN_COLS 16
 #define LIN_PARTS 16
 #define LIN_ROWS 64            // rows of a chunk
 #define LIN_POWERS (LIN_ROWS + 1)
-
-typedef float floatx4 __attribute__((ext_vector_type(4)));
+#define LIN_MIDDLE 32          // a channel decay's narrow row comes in steps of this many
 
 __device__ __forceinline__ floatx4 mfma_f32(float a, float b, floatx4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
@@ -70,8 +71,10 @@ struct LinArgs {
   const int* chunks;    // [chunks, 2]: first row, rows
   float* before;        // [chunks, heads, dv, dk]: a chunk's own sum, then the state in front of it
   // channel decay (powers are then unused)
-  const float* z;       // [rows, ldz]: heads x dk
-  int ldz;
+  int m_off, middle;    // the narrow row: columns m_off .. + middle of y (a multiple of LIN_MIDDLE, filled up with zeros)
+  int rank;             // what of it is not filling
+  const void* w_up;     // [heads x dk, middle], of y's type
+  const float* b_up;    // [heads x dk]
   float inv_tau;
   float* chunk_decay;   // [chunks, heads, dk]: the product of a chunk's alphas
 };
@@ -98,6 +101,24 @@ template <>
 __device__ __forceinline__ float lin_act<bf16_t>(float z, int silu) {
   return silu ? z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)) : z;
 }
+
+template <typename T>
+struct Raw4;  // four neighbouring elements as they lie in memory
+template <>
+struct Raw4<float> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* p) { v = *(const float4*)p; }
+  __device__ __forceinline__ float get(int e) const { return e == 0 ? v.x : e == 1 ? v.y : e == 2 ? v.z : v.w; }
+};
+template <>
+struct Raw4<bf16_t> {
+  uint2 v;
+  __device__ __forceinline__ void load(const bf16_t* p) { v = *(const uint2*)p; }
+  __device__ __forceinline__ float get(int e) const {
+    const uint32_t w = e < 2 ? v.x : v.y;
+    return __uint_as_float((e & 1) ? (w & 0xffff0000u) : (w << 16));
+  }
+};
 
 // thread = cw * 16 + part: column blockIdx.z * 16 + cw, state rows part * E .. + E. C: rows staged at a time
 template <typename T, int E, int C, bool ROT, bool CHAN>
@@ -144,6 +165,8 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
   const T* y = (const T*)A.y;
   const int half = A.rot >> 1;
   const int pos0 = ROT ? A.positions[lo] : 0;
+  // four entries of the narrow row per load where it lies on them
+  const bool mid_wide = CHAN && ((A.ld | A.m_off) & 3) == 0 && ((uintptr_t)A.y % (4 * sizeof(T))) == 0 && ((uintptr_t)A.w_up % (4 * sizeof(T))) == 0;
   const float d = CHAN ? 0.f : A.powers[(size_t)h * LIN_POWERS + 1];
   const size_t q_at = (size_t)A.q_off + (size_t)h * dk, k_at = (size_t)A.k_off + (size_t)h * dk;
   const size_t v_at = (size_t)A.v_off + (size_t)h * A.dv + col0;
@@ -177,7 +200,22 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
         if (C * NP % 256 && idx >= C * NP) break;
         const int t = idx / NP, i = idx % NP;
         const bool own = t < have && i < dk;
-        const float z = A.z[(size_t)(lo + r0 + (own ? t : 0)) * A.ldz + (size_t)h * dk + (own ? i : 0)];
+        const T* m = y + (size_t)(lo + r0 + (own ? t : 0)) * A.ld + A.m_off;
+        const T* w = (const T*)A.w_up + ((size_t)h * dk + (own ? i : 0)) * A.middle;
+        float z = A.b_up[(size_t)h * dk + (own ? i : 0)];
+        if (mid_wide) {
+          for (int k0 = 0; k0 < A.rank; k0 += 16) {
+            Raw4<T> mu[4], wu[4];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) mu[k].load(m + k0 + 4 * k), wu[k].load(w + k0 + 4 * k);
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) z = fmaf(mu[k].get(e), wu[k].get(e), z);
+          }
+        } else {
+          for (int k = 0; k < A.rank; ++k) z = fmaf(ldf(m, k), ldf(w, k), z);
+        }
         sm[t * ROWF + 2 * NP + i] = own ? channel_alpha<T>(z, A.inv_tau) : 0.f;
       }
     }
@@ -215,24 +253,6 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinArgs A) {
 
 // ---------------------------------------------------------------------------------------------------------------------
 // the chunked form: dk and dv in multiples of 16 up to 256, rot in multiples of 8, rows and offsets on 4 elements
-
-template <typename T>
-struct Raw4;  // four neighbouring elements as they lie in memory
-template <>
-struct Raw4<float> {
-  float4 v;
-  __device__ __forceinline__ void load(const float* p) { v = *(const float4*)p; }
-  __device__ __forceinline__ float get(int e) const { return e == 0 ? v.x : e == 1 ? v.y : e == 2 ? v.z : v.w; }
-};
-template <>
-struct Raw4<bf16_t> {
-  uint2 v;
-  __device__ __forceinline__ void load(const bf16_t* p) { v = *(const uint2*)p; }
-  __device__ __forceinline__ float get(int e) const {
-    const uint32_t w = e < 2 ? v.x : v.y;
-    return __uint_as_float((e & 1) ? (w & 0xffff0000u) : (w << 16));
-  }
-};
 
 // Two groups of four entries of a q or k head that the same thread brings in: entries i1 .. + 4 and i2 .. + 4. Below rot / 2
 // they are the two sides of four turned pairs, beyond it neighbours that pass unturned.
@@ -567,6 +587,34 @@ struct TileProducts {
   }
 };
 
+// z of a channel decay for 16 channels (from channel row `w` of W_up on) and 16 rows (a lane holds the one at `m`): lane l gets
+// row l % 16, channels 4 (l / 16) .. + 4, which is how a product of [channels x middle] and [middle x rows] leaves them
+template <typename T>
+struct DecayInput;
+template <>
+struct DecayInput<bf16_t> {
+  static __device__ __forceinline__ floatx4 make(const bf16_t* w, const bf16_t* m, int middle, int l16, int g, floatx4 z) {
+    for (int k0 = 0; k0 < middle; k0 += LIN_MIDDLE) {
+      const u32x4 a = *(const u32x4*)(w + (size_t)l16 * middle + k0 + 8 * g);
+      const u32x4 b = *(const u32x4*)(m + k0 + 8 * g);
+      z = mfma16(a, b, z);
+    }
+    return z;
+  }
+};
+template <>
+struct DecayInput<float> {
+  static __device__ __forceinline__ floatx4 make(const float* w, const float* m, int middle, int l16, int g, floatx4 z) {
+    for (int k0 = 0; k0 < middle; k0 += 16) {
+      const floatx4 a = *(const floatx4*)(w + (size_t)l16 * middle + k0 + 4 * g);
+      const floatx4 b = *(const floatx4*)(m + k0 + 4 * g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) z = mfma_f32(a[e], b[e], z);
+    }
+    return z;
+  }
+};
+
 // A wave stages the rows of tile wave % 4 in every other group of 16 channels from wave / 4 on; lane l: row l % 16, channels
 // 4 (l / 16) .. + 4 of the group.
 // grid (chunk, head, 128 value columns), eight waves, as linear_local
@@ -592,12 +640,13 @@ __global__ __launch_bounds__(512) void linear_channel_local_kernel(LinArgs A) {
   const bool on = row < have;
   const size_t at = (size_t)(lo + min(row, have - 1));  // rows beyond the chunk's are read from its last one and dropped
   Raw4<T> ku[NB], vu[4];
-  float4 zu[NB];
+  floatx4 zu[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
-    const int i = min((b0 + 2 * b) * 16, dk - 16) + 4 * g;
+    const int i0 = min((b0 + 2 * b) * 16, dk - 16), i = i0 + 4 * g;
     ku[b].load(y + at * A.ld + A.k_off + (size_t)h * dk + i);
-    zu[b] = *(const float4*)(A.z + at * A.ldz + (size_t)h * dk + i);
+    zu[b] = DecayInput<T>::make((const T*)A.w_up + ((size_t)h * dk + i0) * A.middle, y + at * A.ld + A.m_off, A.middle, l16, g,
+                                *(const floatx4*)(A.b_up + (size_t)h * dk + i));
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
@@ -607,12 +656,11 @@ __global__ __launch_bounds__(512) void linear_channel_local_kernel(LinArgs A) {
   float u[NB][4];
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
-    const float zz[4] = {zu[b].x, zu[b].y, zu[b].z, zu[b].w};
     float tot[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       TileProducts tp;
-      tp.start(on ? channel_alpha<T>(zz[e], A.inv_tau) : 1.0f);
+      tp.start(on ? channel_alpha<T>(zu[b][e], A.inv_tau) : 1.0f);
       tp.widen<1>(l16);
       tp.widen<2>(l16);
       tp.widen<4>(l16);
@@ -718,20 +766,20 @@ __global__ __launch_bounds__(512) void linear_channel_outputs_kernel(LinArgs A) 
   {
     const size_t at = (size_t)(lo + min(row, have - 1));
     Raw4<T> qu[NB], ku[NB];
-    float4 zu[NB];
+    floatx4 zu[NB];
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
-      const int i = min((b0 + 2 * b) * 16, dk - 16) + 4 * g;
+      const int i0 = min((b0 + 2 * b) * 16, dk - 16), i = i0 + 4 * g;
       qu[b].load(y + at * A.ld + A.q_off + (size_t)h * dk + i);
       ku[b].load(y + at * A.ld + A.k_off + (size_t)h * dk + i);
-      zu[b] = *(const float4*)(A.z + at * A.ldz + (size_t)h * dk + i);
+      zu[b] = DecayInput<T>::make((const T*)A.w_up + ((size_t)h * dk + i0) * A.middle, y + at * A.ld + A.m_off, A.middle, l16, g,
+                                  *(const floatx4*)(A.b_up + (size_t)h * dk + i));
     }
     floatx4 acc1 = {0.f, 0.f, 0.f, 0.f}, acc2 = acc1, acc4 = acc1, acc8 = acc1;
     float own = 0.f;  // q_i . k_i
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
       const int i = (b0 + 2 * b) * 16 + 4 * g;
-      const float zz[4] = {zu[b].x, zu[b].y, zu[b].z, zu[b].w};
       const bool in = on && i < dk;
       float q[4], k[4];
       TileProducts tp[4];
@@ -740,7 +788,7 @@ __global__ __launch_bounds__(512) void linear_channel_outputs_kernel(LinArgs A) 
         q[e] = in ? lin_act<T>(qu[b].get(e), A.silu) : 0.f;
         k[e] = in ? lin_act<T>(ku[b].get(e), A.silu) * A.k_scale : 0.f;
         own = fmaf(q[e], k[e], own);
-        tp[e].start(on ? channel_alpha<T>(zz[e], A.inv_tau) : 1.0f);
+        tp[e].start(on ? channel_alpha<T>(zu[b][e], A.inv_tau) : 1.0f);
       }
       level_product<1>(q, k, tp, l16, acc1);
       level_product<2>(q, k, tp, l16, acc2);
@@ -896,29 +944,29 @@ static int check_args(const char* name, const LinArgs& A, int n_requests) {
     JLLM_FAIL("%s: short rows", name);
   if (A.rot < 0 || A.rot % 2 || A.rot > A.dk || (A.rot && (!A.cos_t || !A.sin_t || !A.positions)))
     JLLM_FAIL("%s: a rotary width of %d for heads of %d", name, A.rot, A.dk);
-  if ((A.z == nullptr) == (A.powers == nullptr)) JLLM_FAIL("%s: a decay per head or per channel", name);
-  if (A.z && (A.ldz < A.heads * A.dk || !(A.inv_tau > 0.f) || A.rot))
-    JLLM_FAIL("%s: decay rows of %d for %d heads of %d (1 / tau %g, rotary width %d)", name, A.ldz, A.heads, A.dk, (double)A.inv_tau, A.rot);
+  if ((A.w_up == nullptr) == (A.powers == nullptr)) JLLM_FAIL("%s: a decay per head or per channel", name);
+  if (A.w_up && (!A.b_up || A.middle <= 0 || A.middle % LIN_MIDDLE || A.rank <= 0 || A.rank > A.middle || A.m_off < 0 || A.ld < A.m_off + A.middle || !(A.inv_tau > 0.f) || A.rot))
+    JLLM_FAIL("%s: a channel decay from columns %d .. + %d of rows of %d (1 / tau %g, rotary width %d)", name, A.m_off, A.middle, A.ld, (double)A.inv_tau, A.rot);
   return 0;
 }
 
 extern "C" int jllm_linear_scan(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
                                 const float* cos_t, const float* sin_t, int rot, int silu, float k_scale, const float* powers,
                                 float* state, float* out, int ldo, const int* row_req, const int* state_slots, int n_rows,
-                                int n_requests, int heads, int dk, int dv, const float* z, int ldz, float inv_tau,
-                                hipStream_t stream) {
+                                int n_requests, int heads, int dk, int dv, int m_off, int middle, int rank, const void* w_up,
+                                const float* b_up, float inv_tau, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, row_req, state_slots,
-            n_rows, heads, dk, dv, nullptr, nullptr, nullptr, z, ldz, inv_tau, nullptr};
+            n_rows, heads, dk, dv, nullptr, nullptr, nullptr, m_off, middle, rank, w_up, b_up, inv_tau, nullptr};
   if (check_args("linear_scan", A, n_requests) != 0) return -1;
   dim3 grid(n_requests, heads, (dv + LIN_COLS - 1) / LIN_COLS);
   const int per_lane = (dk + LIN_PARTS - 1) / LIN_PARTS;
   const bool few = n_rows <= 2 * n_requests;
 #define LIN_LAUNCH(E)                                                             \
   do {                                                                            \
-    if (z && few)                                                                 \
+    if (w_up && few)                                                              \
       linear_scan_kernel<T, E, 2, false, true><<<grid, 256, 0, stream>>>(A);      \
-    else if (z)                                                                   \
+    else if (w_up)                                                                \
       linear_scan_kernel<T, E, 16, false, true><<<grid, 256, 0, stream>>>(A);     \
     else if (few && rot)                                                          \
       linear_scan_kernel<T, E, 2, true, false><<<grid, 256, 0, stream>>>(A);      \
@@ -946,16 +994,16 @@ extern "C" int jllm_linear_scan(const void* y, int ld, int q_off, int k_off, int
 
 // Returns 1 (declined) for sizes that the chunked form does not take. requests [n_requests, 3]: first row, rows, first
 // chunk; chunks [n_chunks, 2]: first row, rows (at most 64, of one request, in order); before: fp32 [n_chunks, heads, dv, dk];
-// with z (a channel decay, powers null) chunk_decay: fp32 [n_chunks, heads, dk]
+// with w_up (a channel decay, powers null) chunk_decay: fp32 [n_chunks, heads, dk]
 extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, int v_off, int dtype, const int* positions,
                                   const float* cos_t, const float* sin_t, int rot, int silu, float k_scale,
                                   const float* powers, float* state, float* out, int ldo, const int* requests,
                                   const int* chunks, int n_chunks, float* before, const int* state_slots, int n_rows,
-                                  int n_requests, int heads, int dk, int dv, const float* z, int ldz, float inv_tau,
-                                  float* chunk_decay, hipStream_t stream) {
+                                  int n_requests, int heads, int dk, int dv, int m_off, int middle, int rank, const void* w_up,
+                                  const float* b_up, float inv_tau, float* chunk_decay, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   LinArgs A{y, ld, q_off, k_off, v_off, positions, cos_t, sin_t, rot, silu, k_scale, powers, state, out, ldo, nullptr, state_slots,
-            n_rows, heads, dk, dv, requests, chunks, before, z, ldz, inv_tau, chunk_decay};
+            n_rows, heads, dk, dv, requests, chunks, before, m_off, middle, rank, w_up, b_up, inv_tau, chunk_decay};
   if (check_args("linear_chunks", A, n_requests) != 0) return -1;
   if (n_chunks < n_requests || n_chunks > n_rows || !requests || !chunks || !before) JLLM_FAIL("linear_chunks: %d chunks of %d rows of %d requests", n_chunks, n_rows, n_requests);
   const size_t bytes4 = dtype == JLLM_F32 ? 16 : 8;
@@ -964,13 +1012,15 @@ extern "C" int jllm_linear_chunks(const void* y, int ld, int q_off, int k_off, i
       (rot && (((uintptr_t)cos_t & 15) || ((uintptr_t)sin_t & 15))))
     return 1;
   if (n_requests > 65535) return 1;
-  if (z && ((ldz & 3) || ((uintptr_t)z & 15) || ((uintptr_t)chunk_decay & 15))) return 1;
-  if (z && !chunk_decay) JLLM_FAIL("linear_chunks: no place for the chunks' decays");
+  const int per16 = dtype == JLLM_F32 ? 4 : 8;  // elements in 16 bytes
+  if (w_up && (ld % per16 || m_off % per16 || ((uintptr_t)y & 15) || ((uintptr_t)w_up & 15) || ((uintptr_t)b_up & 15) || ((uintptr_t)chunk_decay & 15)))
+    return 1;
+  if (w_up && !chunk_decay) JLLM_FAIL("linear_chunks: no place for the chunks' decays");
   const dim3 lgrid(n_chunks, heads, (dv + LIN_LOCAL_COLS - 1) / LIN_LOCAL_COLS), cgrid((unsigned)(((size_t)dk * dv / 4 + 255) / 256), heads, n_requests), ogrid(n_chunks, heads);
   int rc = 0;
 #define LIN_CHUNKS(DT)                                                                     \
   do {                                                                                     \
-    if (z) {                                                                               \
+    if (w_up) {                                                                            \
       linear_channel_local_kernel<T, DT><<<lgrid, 512, 0, stream>>>(A);                    \
       linear_combine_kernel<true><<<cgrid, 256, 0, stream>>>(A);                           \
       rc = launch_channel_outputs<T, DT>(ogrid, stream, A);                                \

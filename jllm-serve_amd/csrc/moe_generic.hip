@@ -340,6 +340,75 @@ __global__ __launch_bounds__(64) void moe_router_kernel(const float* __restrict_
       weights[(size_t)t * top + k] = normalize ? weights[(size_t)t * top + k] / (sum + 1e-20f) * scale : weights[(size_t)t * top + k] * scale;
 }
 
+// The same for experts in one group, up to 256 of them: a lane keeps its experts' scores in registers (expert lane + 64 j),
+// a choice is one reduction over the wave, and nothing passes through LDS.
+template <typename TC, int J>
+__global__ __launch_bounds__(64) void moe_router_wave_kernel(const float* __restrict__ z, int ldz, const TC* __restrict__ correction,
+                                                            int E, int top, float scale, int* __restrict__ chosen,
+                                                            float* __restrict__ weights, int softmax, int normalize) {
+  const int t = blockIdx.x, lane = threadIdx.x;
+  float zz[J], s[J], choice[J];
+#pragma unroll
+  for (int j = 0; j < J; ++j) {
+    const int e = lane + 64 * j;
+    zz[j] = e < E ? z[(size_t)t * ldz + e] : -INFINITY;
+    choice[j] = correction && e < E ? ldf(correction, e) : 0.f;
+  }
+  if (softmax) {
+    float m = zz[0];
+#pragma unroll
+    for (int j = 1; j < J; ++j) m = fmaxf(m, zz[j]);
+    m = wave_max(m);
+    float d = 0.f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      s[j] = lane + 64 * j < E ? expf(zz[j] - m) : 0.f;
+      d += s[j];
+    }
+    d = wave_sum(d);
+#pragma unroll
+    for (int j = 0; j < J; ++j) s[j] = s[j] / d;
+  } else {
+#pragma unroll
+    for (int j = 0; j < J; ++j) s[j] = 1.0f / (1.0f + expf(-zz[j]));
+  }
+#pragma unroll
+  for (int j = 0; j < J; ++j) choice[j] = lane + 64 * j < E ? s[j] + choice[j] : -INFINITY;
+  float sum = 0.f, mine_w = 0.f;
+  int mine_e = 0;
+  for (int k = 0; k < top; ++k) {
+    float bv = -INFINITY, bs = 0.f;
+    int bi = 0x7fffffff;
+#pragma unroll
+    for (int j = 0; j < J; ++j)  // ascending expert: the lowest among equals stays
+      if (choice[j] > bv) bv = choice[j], bi = lane + 64 * j, bs = s[j];
+    float v = bv;
+    int i = bi;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(v, o, 64);
+      const int oi = __shfl_xor(i, o, 64);
+      if (ov > v || (ov == v && oi < i)) v = ov, i = oi;
+    }
+    i = i < E ? i : 0;  // (only where a score is not a number: then nothing is larger than anything)
+    bs = __shfl(bs, i & 63, 64);
+    sum += bs;
+    if (lane == (k & 63)) mine_w = bs, mine_e = i;
+#pragma unroll
+    for (int j = 0; j < J; ++j)
+      if (lane + 64 * j == i) choice[j] = -INFINITY;
+    if ((k & 63) == 63 || k + 1 == top) {  // the choices of these 64 steps (weights raw while more than that many follow)
+      const int k0 = k & ~63;
+      if (lane <= k - k0) chosen[(size_t)t * top + k0 + lane] = mine_e;
+      if (lane <= k - k0) weights[(size_t)t * top + k0 + lane] = mine_w;
+    }
+  }
+  for (int k = lane; k < top; k += 64) {  // a lane reads what it wrote itself
+    const float w = top <= 64 ? mine_w : weights[(size_t)t * top + k];
+    weights[(size_t)t * top + k] = normalize ? w / (sum + 1e-20f) * scale : w * scale;
+  }
+}
+
 extern "C" int jllm_moe_router(const float* z, int ldz, const void* correction, int c_dtype, int T, int E, int groups, int keep,
                                int top, float scale, int* chosen, float* weights, int softmax, int group_max, int normalize,
                                hipStream_t stream) {
@@ -349,6 +418,18 @@ extern "C" int jllm_moe_router(const float* z, int ldz, const void* correction, 
     JLLM_FAIL("moe_router: %d experts in %d groups of which %d are kept, for top %d", E, groups, keep, top);
   const size_t smem = (size_t)(2 * E + 2 * groups) * sizeof(float);
   if (smem > 64 * 1024) JLLM_FAIL("moe_router: %d experts are more than this kernel's LDS holds", E);
+  if (groups == 1 && E <= 256) {
+    JLLM_DISPATCH_1(c_dtype, TC, {
+      if (E <= 64)
+        moe_router_wave_kernel<TC, 1><<<T, 64, 0, stream>>>(z, ldz, (const TC*)correction, E, top, scale, chosen, weights, softmax, normalize);
+      else if (E <= 128)
+        moe_router_wave_kernel<TC, 2><<<T, 64, 0, stream>>>(z, ldz, (const TC*)correction, E, top, scale, chosen, weights, softmax, normalize);
+      else
+        moe_router_wave_kernel<TC, 4><<<T, 64, 0, stream>>>(z, ldz, (const TC*)correction, E, top, scale, chosen, weights, softmax, normalize);
+    })
+    JLLM_CHECK_LAUNCH("moe_router");
+    return 0;
+  }
   JLLM_DISPATCH_1(c_dtype, TC, {
     moe_router_kernel<TC><<<T, 64, smem, stream>>>(z, ldz, (const TC*)correction, E, groups, keep, top, scale, chosen, weights, softmax,
                                                    group_max, normalize);

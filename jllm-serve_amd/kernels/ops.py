@@ -81,8 +81,8 @@ def _declare(lib) -> None:
         "jllm_concat_rows": [_P, _P, _I, _I, _P, _I, _I, _P],
         "jllm_ssm_scan": [_P, _I, _P, _I, _I, _I, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P],
         "jllm_gated_group_norm": [_P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P, _I, _I, _I, _I, _F, _P],
-        "jllm_linear_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _P],
-        "jllm_linear_chunks": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _P, _P],
+        "jllm_linear_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P],
+        "jllm_linear_chunks": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _F, _P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P],
         "jllm_rms_seam": [_P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _P, _F, _P, _F, _P, _I, _I, _P, _P, _P, _P],
         "jllm_rms_between": [_P, _I, _I, _P, _I, _P, _I, _I, _F, _F, _P, _F, _P, _P, _I, _P, _F, _P, _I, _I, _P],
         "jllm_token_shift": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
@@ -1571,6 +1571,7 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps
 
 MAX_LINEAR_DIM = 256     # state rows per head that the recurrence keeps in registers (csrc/linear_attention.hip)
 LINEAR_CHUNK = 64        # rows of a chunk of the chunked form
+LINEAR_MIDDLE = 32       # the narrow row of a channel decay comes in steps of this many
 LINEAR_CHUNK_FROM = 24   # a step with a request of at least this many rows takes the chunked form
 
 
@@ -1609,27 +1610,34 @@ def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers
                      positions: Optional[torch.Tensor] = None, cos: Optional[torch.Tensor] = None,
                      sin: Optional[torch.Tensor] = None, rot_dims: int = 0, silu: bool = False, k_scale: float = 1.0,
                      requests: Optional[torch.Tensor] = None, chunks: Optional[torch.Tensor] = None,
-                     decay_rows: Optional[torch.Tensor] = None, tau: float = 1.0) -> torch.Tensor:
+                     decay_off: int = 0, decay_up: Optional[torch.Tensor] = None, decay_bias: Optional[torch.Tensor] = None,
+                     decay_rank: Optional[int] = None, tau: float = 1.0) -> torch.Tensor:
     """Linear attention with a decay over the step's rows, request by request, from and into ``state``
     [slots, heads, dv, dk] (fp32; a head's matrix S [dk, dv] column by column). ``y`` rows hold q and k (heads x dk) and v
     (heads x dv) at the given offsets; with ``silu`` all three pass silu; with ``rot_dims`` the pairs (i, i + rot_dims / 2)
     of every q and k head turn by the table rows of the positions; k is multiplied by ``k_scale``. Per head S <- d S + k
     v^T, o = S^T q with d from ``powers`` (``decay_powers``). Returns o, fp32 [T, heads x dv]. ``requests`` and ``chunks``
     (``linear_chunk_plan`` on the device): the chunked form on the matrix cores (fp32), where the sizes allow it; without
-    them the rows are walked one by one. ``decay_rows`` (fp32 [T, heads x dk], with ``powers`` None): a decay per key channel
-    and token instead, sigmoid(decay_rows)^(1 / tau), on the rows of S (no rotation)."""
-    _dev(y, powers, decay_rows, state, row_req, state_slots, positions, cos, sin, requests, chunks)
+    them the rows are walked one by one. ``decay_up`` (with ``powers`` None): a decay per key channel and token instead, on the
+    rows of S (no rotation): sigmoid(z)^(1 / tau) with z = decay_up m + decay_bias in fp32, m the columns of ``y`` from
+    ``decay_off`` on; ``decay_up`` [heads x dk, middle] is of y's type, its middle a multiple of ``LINEAR_MIDDLE``
+    (filled up with zeros behind the first ``decay_rank``), ``decay_bias`` fp32 [heads x dk]."""
+    _dev(y, powers, decay_up, decay_bias, state, row_req, state_slots, positions, cos, sin, requests, chunks)
     _rows2d(y, "projection rows")
     T = y.shape[0]
     if min(q_off, k_off, v_off) < 0 or max(q_off + heads * dk, k_off + heads * dk, v_off + heads * dv) > y.shape[1]:
         raise KernelError("linear attention: q, k or v lie outside the projection rows")
-    if (powers is None) == (decay_rows is None):
+    if (powers is None) == (decay_up is None):
         raise KernelError("linear attention: a decay per head or per channel")
-    if decay_rows is not None:
-        _rows2d(decay_rows, "decay rows")
-        if decay_rows.dtype != torch.float32 or decay_rows.shape != (T, heads * dk) or not tau > 0 or rot_dims:
-            raise KernelError(f"linear attention: {decay_rows.dtype} decay rows {tuple(decay_rows.shape)} for {(T, heads * dk)}, "
-                              f"tau {tau}, rotary width {rot_dims}")
+    if decay_up is not None:
+        middle = decay_up.shape[1] if decay_up.dim() == 2 else 0
+        if decay_up.dtype != y.dtype or not decay_up.is_contiguous() or decay_up.shape != (heads * dk, middle) or middle % LINEAR_MIDDLE \
+                or middle == 0 or decay_off < 0 or decay_off + middle > y.shape[1] or not tau > 0 or rot_dims:
+            raise KernelError(f"linear attention: a channel decay through {decay_up.dtype} {tuple(decay_up.shape)} from column {decay_off} of "
+                              f"rows of {y.shape[1]}, tau {tau}, rotary width {rot_dims}")
+        if decay_bias is None:
+            raise KernelError("linear attention: a channel decay without its bias")
+        _vec32(decay_bias, heads * dk, "the channel decay's bias")
     elif powers.dtype != torch.float32 or not powers.is_contiguous() or powers.shape != (heads, LINEAR_CHUNK + 1):
         raise KernelError(f"linear attention: the decays' powers must be a contiguous fp32 [{heads}, {LINEAR_CHUNK + 1}] tensor")
     if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 4 or state.shape[1:] != (heads, dv, dk):
@@ -1647,13 +1655,14 @@ def linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, powers
     head = (_ptr(y), y.stride(0), int(q_off), int(k_off), int(v_off), _code(y.dtype), _ptr(positions) if rot_dims else None,
             _ptr(cos) if rot_dims else None, _ptr(sin) if rot_dims else None, int(rot_dims), 1 if silu else 0, float(k_scale),
             _ptr(powers), _ptr(state), _ptr(out), out.stride(0))
-    decay = (_ptr(decay_rows), decay_rows.stride(0) if decay_rows is not None else 0, 1.0 / float(tau))
+    middle = decay_up.shape[1] if decay_up is not None else 0
+    decay = (int(decay_off), middle, middle if decay_rank is None else int(decay_rank), _ptr(decay_up), _ptr(decay_bias), 1.0 / float(tau))
     if requests is not None and chunks is not None and requests.numel() and chunks.numel():
         _i32(requests, 3 * n_requests, "requests of the chunk plan")
         _i32(chunks, 2, "chunks")
         n_chunks = chunks.numel() // 2
         before = torch.empty((n_chunks * heads * dv * dk,), dtype=torch.float32, device=y.device)
-        chunk_decay = torch.empty((n_chunks * heads * dk,), dtype=torch.float32, device=y.device) if decay_rows is not None else None
+        chunk_decay = torch.empty((n_chunks * heads * dk,), dtype=torch.float32, device=y.device) if decay_up is not None else None
         if _try("jllm_linear_chunks", *head, _ptr(requests), _ptr(chunks), n_chunks, _ptr(before), _ptr(state_slots), T,
                 int(n_requests), heads, dk, dv, *decay, _ptr(chunk_decay), _stream()):
             return out

@@ -4,8 +4,9 @@ cache manager's state slots. Nothing is paged and nothing grows with the context
 
 A step is
   1. one product with the stacked weight [W_q | W_k | W_v | W_g] (and, where the token chooses its decays, the narrow W_down
-     of their input, whose second half is a product of its own into fp32 rows),
-  2. the recurrence over each request's rows in order, with the activation, the rotation and k's constant inside
+     of their input),
+  2. the recurrence over each request's rows in order, with the activation, the rotation, k's constant and the second half
+     of the decays' input inside
      (``ops.linear_attention``; its read-out comes back raw, in fp32): row by row for steps of few rows per request, in
      chunks of 64 rows as fp32 matrix products for portions of prompts,
   3. the norm of every head (``ops.heads_finish``, the kernel that ends attention heads too) or of the whole row
@@ -67,7 +68,7 @@ class LinearAttention(Part):
         self.qk_dim = spec.heads * spec.dim
         self.v_dim = spec.heads * spec.vdim
         self.decay_at = 2 * self.qk_dim + 2 * self.v_dim  # the stacked product's columns behind q | k | v | gate
-        self.w_in = self.w_o = self.gain = self.powers = self.w_decay_up = self.b_decay = None
+        self.w_in = self.w_o = self.gain = self.powers = self.w_decay_up = self.b_decay = self.decay_rank = None
 
     def _name(self, which: str) -> str:
         return f"{self.prefix}.{getattr(self.spec.names, which)}"
@@ -88,11 +89,15 @@ class LinearAttention(Part):
     def load(self, get):
         stack = [get(self._name(n)) for n in ("q", "k", "v", "gate") + (("decay_down",) if self.channel else ())]
         if self.channel:
-            self.w_decay_up = get(self._name("decay_up"))
+            up = get(self._name("decay_up"))
             self.b_decay = get(self._name("decay_bias")).float().contiguous()
-            if self.w_decay_up.shape[1] != stack[-1].shape[0]:
+            if up.shape[1] != stack[-1].shape[0]:
                 raise ValueError(f"{self.prefix}: the two halves of the decay's input disagree about their middle: "
-                                 f"{stack[-1].shape[0]} and {self.w_decay_up.shape[1]}")
+                                 f"{stack[-1].shape[0]} and {up.shape[1]}")
+            self.decay_rank = up.shape[1]
+            # the middle filled up with zeros, on both sides, to what the recurrence takes
+            stack[-1] = pad_rows(stack[-1], ops.LINEAR_MIDDLE)
+            self.w_decay_up = pad_rows(up.t().to(self.build.dtype), ops.LINEAR_MIDDLE).t().contiguous()
         dt = stack[0].dtype if all(t.dtype == stack[0].dtype for t in stack) else torch.float32
         self.w_in = pad_rows(torch.cat([t.to(dt) for t in stack], dim=0).contiguous())
         self.w_o = get(self._name("o"))
@@ -131,14 +136,11 @@ class LinearAttention(Part):
         plan = step.plans.get(LinearStepPlanner.key)
         requests = plan.arrays.get("requests") if plan is not None else None
         chunks = plan.arrays.get("chunks") if plan is not None else None
-        decay_rows = None
-        if self.channel:  # what enters the recurrence besides the projections is fp32
-            decay_rows = ops.gemm(y[:, self.decay_at:self.decay_at + self.w_decay_up.shape[1]], self.w_decay_up, bias=self.b_decay,
-                                  out_dtype=torch.float32, exact=self.build.exact)
         o = ops.linear_attention(y, 0, self.qk_dim, 2 * self.qk_dim, self.powers, slot.state, step.row_req, step.state_slots,
                                  step.n_requests, s.heads, s.dim, s.vdim, positions=step.positions, cos=cos, sin=sin,
                                  rot_dims=rdims, silu=s.activation == "silu", k_scale=s.k_scale, requests=requests, chunks=chunks,
-                                 decay_rows=decay_rows, tau=s.tau)
+                                 decay_off=self.decay_at, decay_up=self.w_decay_up, decay_bias=self.b_decay,
+                                 decay_rank=self.decay_rank, tau=s.tau)
         gate_at = 2 * self.qk_dim + self.v_dim
         gate = y[:, gate_at:gate_at + self.v_dim]
         if s.norm != "whole":
