@@ -88,8 +88,12 @@ __device__ __forceinline__ float channel_alpha<float>(float z, float inv_tau) {
 }
 template <>
 __device__ __forceinline__ float channel_alpha<bf16_t>(float z, float inv_tau) {
+  // the hardware's exp2 and log2. A decay near 1 acts on hundreds of tokens, so what 1 + x loses of a small x = exp(-|z|) is
+  // made good: log(1 + x) = x log(u) / (u - 1) with u = 1 + x as rounded, and x itself where u is 1
   const float z2 = 1.4426950408889634f * z;
-  return __builtin_amdgcn_exp2f((fminf(z2, 0.f) - __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(z2)))) * inv_tau);
+  const float x = __builtin_amdgcn_exp2f(-fabsf(z2)), u = 1.0f + x, d = u - 1.0f;
+  const float l = d == 0.f ? 1.4426950408889634f * x : __builtin_amdgcn_logf(u) * x * __builtin_amdgcn_rcpf(d);
+  return __builtin_amdgcn_exp2f((fminf(z2, 0.f) - l) * inv_tau);
 }
 
 // bf16 inputs: the hardware's exp2 and reciprocal (each within a unit or two of the last place in fp32)

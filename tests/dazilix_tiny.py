@@ -44,7 +44,7 @@ D_A = {
 }
 
 D_B = {
-    "architecture": "Dazilix", "vocab": 288, "width": 128, "norm": {"eps": 1e-4}, "embedding": {"scale": 0.8},
+    "architecture": "Dazilix", "vocab": 288, "width": 128, "norm": {"eps": 1e-4}, "embedding": {"scale": 1.6},
     "layers": [
         _layer(_att(8, 2, 32, 100, 0.2, 16, 5000.0), 16, 3, 64),
         _layer(_gla(3, 64, 48, 4.0), 8, 2, 128),
@@ -78,7 +78,8 @@ CONFIGS = {"DA": (D_A, 61, 8, 5), "DB": (D_B, 62, 16, 24), "DC": (D_C, 63, 4, 1)
 def write_model(folder, cfg, seed, middle=16, std=0.09):
     """A model folder with random weights wide enough that every mechanism moves the logits: the embedding and the pass
     vectors N(0, 0.7), matrices N(0, std) (the attention's q and k gains 1.4 + N(0, 0.3), so that scores have a spread),
-    norms 1 + N(0, 0.3), factors per channel 0.8 + N(0, 0.3), router logits with a spread, and decays from nearly 0 to
+    norms 1 + N(0, 0.3), factors per channel 0.4 + N(0, 0.15), routers whose choice
+    depends on the token but is seldom a close call (weights N(0, 0.08), biases N(0, 2)), and decays from nearly 0 to
     nearly 1 (their bias N(2, 2.5), their matrices N(0, 0.3))."""
     from jllm_serve_amd.weights.random_init import random_source
     from jllm_serve_amd.weights.safetensors_io import write_safetensors
@@ -99,12 +100,14 @@ def write_model(folder, cfg, seed, middle=16, std=0.09):
             tensors[n] = normal((t.shape[0], middle), 0.0, 0.3)
         elif n.endswith("a2.b"):
             tensors[n] = normal(t.shape, 2.0, 2.5)
-        elif n.endswith("router") or n.endswith("router.b"):
-            tensors[n] = normal(t.shape, 0.0, 0.3)
+        elif n.endswith("router"):
+            tensors[n] = normal(t.shape, 0.0, 0.08)
+        elif n.endswith("router.b"):
+            tensors[n] = normal(t.shape, 0.0, 2.0)
         elif n.endswith("q.norm") or n.endswith("k.norm"):
             tensors[n] = normal(t.shape, 1.4, 0.3)
         elif last in ("ls1", "ls2"):
-            tensors[n] = normal(t.shape, 0.8, 0.3)
+            tensors[n] = normal(t.shape, 0.4, 0.15)
         elif last.startswith("norm"):
             tensors[n] = normal(t.shape, 1.0, 0.3)
     os.makedirs(folder, exist_ok=True)
@@ -136,7 +139,14 @@ def tolerance(dtype, ref):
     bits of mantissa can do to single rows (with routers whose choice it can turn); ``typical`` bounds the median over many
     rows, and the float32 run, which takes the same path through cache, state and batching, is held tightly."""
     m = float(ref.abs().max())
-    return 5e-5 * m + 1e-6 if dtype == "float32" else 0.1 * m
+    return 1e-4 * m + 1e-6 if dtype == "float32" else 0.1 * m
+
+
+def turned(dtype, rows):
+    """How many of a whole model's rows may lie beyond ``tolerance``. A router's choice is a step function of its input: in
+    bfloat16 the normed rows carry a rounding of a few parts in a thousand, which turns a close call between two experts
+    here and there, and through states and caches the rows behind it."""
+    return 0 if dtype == "float32" else max(1, rows // 25)
 
 
 def typical(dtype):
